@@ -16,7 +16,7 @@ from typing import Any, Optional
 @dataclass
 class ModelConfig:
     name: str
-    arch: str                       # "llama" | "gpt2" | "mixtral" | "nesizen" | "zinesun" | "lizizen" | "gevipel"
+    arch: str                       # "llama" | "gpt2" | "mixtral" | "nesizen" | "zinesun" | "lizizen" | "gevipel" | "vuladra"
     vocab_size: int
     hidden_size: int
     intermediate_size: int
@@ -104,7 +104,8 @@ class ModelConfig:
                 sum((2 * sp["kv_rank"] + sp["rot_dim"]) * dtype_bytes for sp in runs
                     if sp["type"] == "latent_attention") + \
                 sum(sp["kv_heads"] * (sp["maps"] * sp["dim"] + sp["vdim"]) * dtype_bytes for sp in runs
-                    if sp["type"] in ("biased_attention", "diff_attention", "sloped_attention"))
+                    if sp["type"] in ("biased_attention", "diff_attention", "sloped_attention", "pooled_attention",
+                                      "side_by_side"))
         return 2 * self.num_layers * self.kv_size * dtype_bytes
 
     # ---- (de)serialisation -------------------------------------------------------------
@@ -247,6 +248,31 @@ class ModelConfig:
                    residual_mult=float(js.get("residual_mult", 1.0)))
 
     @classmethod
+    def from_vuladra(cls, js: dict, name: str = "vuladra") -> "ModelConfig":
+        """Map a Vuladra config.json ("architecture": "Vuladra") to ModelConfig: layers with an RMS norm
+        before and after every sublayer, three mixers (sigmoid attention over a window and pooled blocks,
+        "attention"; windowed softmax attention beside linear attention with a constant decay,
+        "parallel"; the selective scan, "mamba1"), dense silu GLUs or routed clamped GLUs with a shared
+        expert, the embedding table as LM head. Every size and per-layer constant is taken from the file."""
+        kinds = {"attention": "pooled_attention", "parallel": "side_by_side", "mamba1": "selective_scan"}
+        specs = []
+        for i, L in enumerate(js["layers"]):
+            if L["type"] not in kinds:
+                raise ValueError(f"layer {i}: Vuladra has no mixer {L['type']!r}")
+            specs.append(layer_spec(i, {**L, "type": kinds[L["type"]]}))
+        mx = lambda key: max([sp.get(key) or 0 for sp in specs] + [0])  # noqa: E731
+        ffs = [sp["ffn"] for sp in specs if sp["ffn"]]
+        moe = [f for f in ffs if f["kind"] == "moe"]
+        shared = [f["shared"]["ff"] for f in moe if f.get("shared")]
+        return cls(name=name, arch="vuladra", vocab_size=int(js["vocab"]), hidden_size=int(js["width"]),
+                   intermediate_size=max([f["ff"] for f in ffs] + shared + [mx("inner"), 0]),
+                   num_layers=len(specs), num_heads=max(mx("heads"), mx("r_heads")), num_kv_heads=max(mx("kv_heads"), 1),
+                   head_dim=max(mx("dim"), mx("vdim"), mx("r_dim"), mx("r_vdim")), max_position=1 << 30,
+                   norm_eps=float(js["norm"]["eps"]), norm="rms", act="silu", pos_emb="none", tie_embeddings=True,
+                   num_experts=max([f["experts"] for f in moe] + [0]),
+                   experts_per_token=max([f["top"] for f in moe] + [0]), layer_specs=specs)
+
+    @classmethod
     def from_model_dir(cls, path, name: Optional[str] = None) -> "ModelConfig":
         """config.json of a model folder -> ModelConfig; the "architecture" / "model_type" key
         chooses the family."""
@@ -261,6 +287,8 @@ class ModelConfig:
             return cls.from_lizizen(js, name=name)
         if family == "gevipel":
             return cls.from_gevipel(js, name=name)
+        if family == "vuladra":
+            return cls.from_vuladra(js, name=name)
         return cls.from_hf(js, name=name)
 
     @classmethod
@@ -313,9 +341,18 @@ def layer_spec(index: int, L: dict) -> dict:
     are the keys as projected, with normed queries and keys, a linear per-head distance bias and the
     query temperature (heads, kv_heads, dim, vdim = dim, scale, window, qt_coef, qt_every); "delta":
     the gated delta rule with short convolutions on its query, key and value rows (heads, kv_heads,
-    dim, vdim, taps). `ffn`: None, or kind "dense" (ff) / "glu" (dense clamped GLU with biases: ff,
-    limit) / "moe" (ff, limit or None for unclamped experts, experts, top)."""
+    dim, vdim, taps); "pooled_attention": attention with sigmoid weights over a sliding window and, before
+    it, the means of blocks of `pool` positions (heads, kv_heads, dim, vdim, scale, window, pool = 0: window
+    only), norms over whole projections, an elementwise output gate; "side_by_side": windowed softmax
+    attention (heads, kv_heads, dim, vdim, scale, window, left_scale) and linear attention with one constant
+    decay per head (r_heads, r_dim, r_vdim, decay, right_scale) on the same input, summed;
+    "selective_scan": a gated state-space layer with a short convolution (inner, state, dt_rank, taps).
+    `ffn`: None, or kind "dense" (ff) / "glu" (dense clamped GLU with biases: ff,
+    limit) / "moe" (ff, limit or None for unclamped experts, experts, top, and for some stacks shared: None or
+    the always-used expert's ff and limit)."""
     m, t = L["mixer"], L["type"]
+    if t in ("pooled_attention", "side_by_side", "selective_scan"):
+        return _vuladra_spec(index, t, m, L.get("mlp"))
     sp = {"index": index, "type": t, "heads": int(m["heads"]), "dim": int(m["dim"]), "vdim": int(m.get("vdim", m["dim"])),
           "kv_from": None, "kv_heads": 0, "maps": 1}
     if t == "biased_attention":
@@ -392,7 +429,68 @@ def layer_spec(index: int, L: dict) -> dict:
     return sp
 
 
+def _attention_sizes(index: int, m: dict) -> dict:
+    """Heads, sizes, scale and window (NO_WINDOW when absent) of a grouped attention without rotation."""
+    H, D = int(m["heads"]), int(m["dim"])
+    mask = m.get("mask") or {}
+    sp = {"heads": H, "kv_heads": int(m.get("kv_heads", H)), "dim": D, "vdim": int(m.get("vdim", D)),
+          "scale": float(m.get("scale", D ** -0.5)), "window": int(mask.get("size", 1 << 30)),
+          "pool": int(mask.get("pool") or 0)}
+    if sp["kv_heads"] < 1 or H % sp["kv_heads"] or min(D, sp["vdim"], sp["window"]) < 1 or sp["pool"] < 0:
+        raise ValueError(f"layer {index}: bad attention sizes")
+    return sp
+
+
+def _vuladra_spec(index: int, t: str, m: dict, f: Optional[dict]) -> dict:
+    sp = {"index": index, "type": t, "kv_from": None, "maps": 1, "heads": 0, "kv_heads": 0, "dim": 0, "vdim": 0}
+    if t == "pooled_attention":
+        sp.update(_attention_sizes(index, m))
+    elif t == "side_by_side":
+        r = m["right"]
+        sp.update(_attention_sizes(index, m["left"]))
+        sp.update(r_heads=int(r["heads"]), r_dim=int(r["dim"]), r_vdim=int(r.get("vdim", r["dim"])),
+                  decay=[float(x) for x in r["decay"]], left_scale=float(m.get("left_scale", 1.0)),
+                  right_scale=float(m.get("right_scale", 1.0)))
+        if sp["pool"] or sp["r_heads"] < 1 or len(sp["decay"]) != sp["r_heads"] or min(sp["r_dim"], sp["r_vdim"]) < 1:
+            raise ValueError(f"layer {index}: bad sizes of the parallel mixers")
+    else:
+        sp.update(inner=int(m["inner"]), state=int(m["state"]), dt_rank=int(m["dt_rank"]), taps=int(m.get("conv", 1)))
+        if min(sp["inner"], sp["state"], sp["dt_rank"], sp["taps"]) < 1:
+            raise ValueError(f"layer {index}: bad selective-scan sizes")
+    lim = lambda d: float("inf") if d.get("limit") is None else float(d["limit"])  # noqa: E731
+    if f is None:
+        sp["ffn"] = None
+    elif f["kind"] == "dense":
+        sp["ffn"] = {"kind": "dense", "ff": int(f["ff"])}
+    elif f["kind"] == "moe":
+        sh = f.get("shared")
+        sp["ffn"] = {"kind": "moe", "ff": int(f["expert"]["ff"]), "limit": lim(f["expert"]),
+                     "experts": int(f["router"]["experts"]), "top": int(f["router"]["top"]),
+                     "shared": {"ff": int(sh["ff"]), "limit": lim(sh)} if sh else None}
+        if not 1 <= sp["ffn"]["top"] <= sp["ffn"]["experts"]:
+            raise ValueError(f"layer {index}: top must be in 1..experts")
+    else:
+        raise ValueError(f"layer {index}: unknown feed-forward kind {f['kind']!r}")
+    return sp
+
+
 def layer_spec_params(h: int, sp: dict) -> int:
+    if sp["type"] in ("pooled_attention", "side_by_side", "selective_scan"):
+        H, G, D, Dv = sp["heads"], sp["kv_heads"], sp["dim"], sp["vdim"]
+        n = h * (H * D + G * (D + Dv)) + H * Dv * h
+        if sp["type"] == "pooled_attention":
+            n += (H + G) * D + H + h * H * Dv
+        elif sp["type"] == "side_by_side":
+            n += sp["r_heads"] * (2 * h * sp["r_dim"] + 3 * h * sp["r_vdim"] + sp["r_vdim"])
+        else:
+            c, N, r = sp["inner"], sp["state"], sp["dt_rank"]
+            n = 3 * h * c + c * (sp["taps"] + 1) + c * (r + 2 * N) + c * r + c + c * N + c
+        f = sp["ffn"]
+        if f and f["kind"] == "dense":
+            n += 3 * h * f["ff"]
+        elif f:
+            n += f["experts"] * (3 * h * f["ff"] + h) + (3 * h * f["shared"]["ff"] if f["shared"] else 0)
+        return n + (4 if f else 2) * h
     H, D, Dv = sp["heads"], sp["dim"], sp["vdim"]
     if sp["type"] == "attention":
         n = h * H * D + H * Dv * h + H

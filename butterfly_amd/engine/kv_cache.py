@@ -3,6 +3,8 @@
 Layout per local layer (models/transformer.py allocate_kv_cache):
   K [num_blocks, kv_heads_local, block_size, head_dim]   (rows contiguous: QK^T operand)
   V [num_blocks, kv_heads_local, head_dim, block_size]   (transposed: PV operand)
+A layer may keep further per-page tensors behind the pair (first dimension num_blocks), e.g. the mean
+keys and values of pooled blocks: they are copied, reused and freed with the page.
 Elements are the model dtype or, with EngineConfig.kv_cache_dtype="fp8", FP8 e4m3
 (torch.float8_e4m3fn, written and read by the HIP kernels: csrc/include/bfly_kv.h).
 Capacity is sized from the HBM left after weights and activations (SURVEY.md §2.7 A14:
@@ -54,12 +56,12 @@ class KVCache:
         return self.num_blocks * self.block_size
 
     def bytes(self) -> int:
-        return sum(k.numel() * k.element_size() + v.numel() * v.element_size() for k, v in self.layers) + \
+        return sum(t.numel() * t.element_size() for layer in self.layers for t in layer) + \
             sum(t.numel() * t.element_size() for t in self.state)
 
     def copy_blocks(self, pairs: list) -> None:
         """Copy-on-write page copies (src -> dst) before a step that writes to a forked page."""
         for src, dst in pairs:
-            for k, v in self.layers:
-                k[dst].copy_(k[src])
-                v[dst].copy_(v[src])
+            for layer in self.layers:
+                for t in layer:
+                    t[dst].copy_(t[src])

@@ -3,13 +3,16 @@ Nesizen, a heterogeneous stack of attention / gated-linear-attention layers (mod
 Zinesun, latent-attention layers on a post-norm residual (models/zinesun.py), and Lizizen, parallel
 layers with a token shift over distance-biased and differential attention (models/lizizen.py), and
 Gevipel, sandwich-normed layers over sloped window attention, the gated delta rule and latent
-attention with a sink, with routed plain experts (models/gevipel.py)."""
+attention with a sink, with routed plain experts (models/gevipel.py), and Vuladra, RMS-sandwiched layers
+over sigmoid attention with pooled blocks, windowed attention beside decayed linear attention, and the
+selective scan, with routed and shared clamped GLUs (models/vuladra.py)."""
 from .shard import LocalDims, Shard, local_dims  # noqa: F401
 from .transformer import LogicalParam, TransformerLM  # noqa: F401
 from .nesizen import NesizenLM  # noqa: F401
 from .zinesun import ZinesunLM  # noqa: F401
 from .lizizen import LizizenLM  # noqa: F401
 from .gevipel import GevipelLM  # noqa: F401
+from .vuladra import VuladraLM  # noqa: F401
 
 
 class LlamaForCausalLM(TransformerLM):
@@ -25,7 +28,8 @@ class GPT2LMHeadModel(TransformerLM):
 
 
 _ARCH = {"llama": LlamaForCausalLM, "mixtral": MixtralForCausalLM, "gpt2": GPT2LMHeadModel,
-         "nesizen": NesizenLM, "zinesun": ZinesunLM, "lizizen": LizizenLM, "gevipel": GevipelLM}
+         "nesizen": NesizenLM, "zinesun": ZinesunLM, "lizizen": LizizenLM, "gevipel": GevipelLM,
+         "vuladra": VuladraLM}
 
 
 def supports_f32(arch: str) -> bool:

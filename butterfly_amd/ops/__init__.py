@@ -841,7 +841,9 @@ def row_seq(row_cu, T: int):
 
 def attn_window_paged(q, k_cache, v_cache, tables, row_cu, positions, scale: float, window: int, keep_first: int,
                       sink, row_map=None, out=None, fold_heads: bool = False, out_scale=None, chunk: int = 0,
-                      softcap: float = 0.0, dist_bias=None, q_temp=None, maps: int = 1, out_dtype=None):
+                      softcap: float = 0.0, dist_bias=None, q_temp=None, maps: int = 1, out_dtype=None,
+                      sigmoid: bool = False, key_bias=None, pool=None, gate=None, out_mul: float = 1.0,
+                      dv_out: int = 0):
     """Windowed attention of packed rows over the paged cache with kept first positions and a
     sink logit (mixers.hip attn_window_paged_kernel; sink None: an ordinary softmax). `row_map`:
     ops.row_seq(row_cu, T), when the caller already has it. `out_scale` [T, H] f32 multiplies
@@ -857,11 +859,21 @@ def attn_window_paged(q, k_cache, v_cache, tables, row_cu, positions, scale: flo
     (counted from position 0). `maps` > 1: the key cache holds `maps` key heads per value head
     (K [blocks, G * maps, BS, D]), the query heads are ordered (head, map), and query head (h, m)
     reads key head (g(h), m) and value head g(h): several attention maps over the same values.
-    `out_dtype` torch.float32: the output keeps the f32 accumulator."""
+    `out_dtype` torch.float32: the output keeps the f32 accumulator.
+
+    Extended form, dv_out > 0: the first dv_out values of every head go to out [T, H * dv_out] (may be a
+    view into wider rows), times out_mul, times sigmoid(gate) (gate [T, H * dv_out] rows; None: no gate),
+    and the query heads of a key / value head share a tile. With it `sigmoid`: the weight of a visible
+    key is sigmoid(s + key_bias[h]) (key_bias [H] f32), not normalised over the keys; `pool` (P, k_pool,
+    v_pool): beside the tokens of its window a row at p sees every block of P positions that ends at or
+    before p - window, through the block's mean key and value (pool_blocks_)."""
     if not _gpu(q):
         return ref.attn_window_paged(q, k_cache, v_cache, tables, row_cu, positions, scale, window, keep_first, sink, out,
-                                     out_scale, chunk, softcap, dist_bias, q_temp, maps, out_dtype)
-    if out is None:
+                                     out_scale, chunk, softcap, dist_bias, q_temp, maps, out_dtype, sigmoid, key_bias, pool,
+                                     gate, out_mul, dv_out)
+    if out is None and dv_out:
+        out = _empty(q.shape[0], q.shape[1] * dv_out, dtype=out_dtype or q.dtype, device=q.device)
+    elif out is None:
         out = _empty(q.shape[0], q.shape[1], v_cache.shape[2], dtype=out_dtype or q.dtype, device=q.device)
     if row_map is None:
         row_map = row_seq(row_cu, q.shape[0])
@@ -874,7 +886,9 @@ def attn_window_paged(q, k_cache, v_cache, tables, row_cu, positions, scale: flo
     qc, qe = q_temp if q_temp is not None else (0.0, 1)
     torch.ops.bfly.attn_window_paged(q, k_cache, v_cache, tables, row_map, row_cu, positions, float(scale), int(window),
                                      int(keep_first), sink, out_scale, bool(fold_heads), part, out, int(chunk),
-                                     float(softcap), da, db, float(qc), int(qe), int(maps))
+                                     float(softcap), da, db, float(qc), int(qe), int(maps), bool(sigmoid), key_bias,
+                                     *((int(pool[0]), pool[1], pool[2]) if pool is not None else (0, None, None)), gate,
+                                     float(out_mul), int(dv_out))
     return out
 
 
@@ -919,16 +933,17 @@ def moe_route_scores(x, wr, top_k: int, scoring: str = "softmax", renorm: bool =
 
 
 def moe_glu_ffn(x, topk_ids, topk_w, gate_up_w, down_w, limit: float, alpha: float, up_offset: float = 1.0,
-                scale_input: bool = True, plain_act=None):
+                scale_input: bool = True, plain_act=None, addend=None):
     """Routed GLU experts y = g' sigmoid(alpha g') (u' + up_offset) with g', u' clamped at `limit`
     (inf, alpha 1, up_offset 0: the plain silu GLU). scale_input: each expert runs on (routing
     score * x) and the outputs are summed; otherwise it runs on x and the sum is weighted by the
     scores. See ops.reference.moe_glu_ffn. gate_up_w [E, 2F, H], down_w [E, H, F]. plain_act
     "relu2": experts without a gate, y = relu(W_up h)^2 with gate_up_w [E, F, H] (limit, alpha and
-    up_offset unused)."""
+    up_offset unused). addend [T, H] (rows may be strided): added to the f32 sum, e.g. a shared
+    expert's output."""
     if not _gpu(x):
         return ref.moe_glu_ffn(x, topk_ids, topk_w, gate_up_w, down_w, limit, alpha, None, up_offset, scale_input,
-                               plain_act)
+                               plain_act, addend)
     T, H = x.shape
     E, F = gate_up_w.shape[0], down_w.shape[2]
     TK = T * topk_ids.shape[1]
@@ -939,7 +954,7 @@ def moe_glu_ffn(x, topk_ids, topk_w, gate_up_w, down_w, limit: float, alpha: flo
     y = _arena.get(dev, "moe_glu_y", TK * H, torch.float32)
     out = _empty(T, H, dtype=x.dtype, device=dev)
     torch.ops.bfly.moe_glu_ffn(x, topk_ids, topk_w, gate_up_w, down_w, float(limit), float(alpha), float(up_offset),
-                               bool(scale_input), work, hmid, y, out, ACTS[plain_act or "none"])
+                               bool(scale_input), work, hmid, y, out, ACTS[plain_act or "none"], addend)
     return out
 
 
@@ -1192,32 +1207,50 @@ def _glu_fused_ok(M: int, N: int, K: int) -> bool:
 # ---------------------------------------------------------------------------------------
 # Sandwich-norm residual stacks with a gated delta rule (csrc/kernels/delta.hip)
 # ---------------------------------------------------------------------------------------
-def post_norm_add_norm(x, y, norm_w, norm_b, eps: float, mult: float, extra, norm2_w, norm2_b, out_dtype):
+def post_norm_add_norm(x, y, norm_w, norm_b, eps: float, mult: float, extra, norm2_w, norm2_b, out_dtype,
+                       rms: bool = False):
     """One launch between two sublayers of a stack with norms on both sides of every sublayer:
     x <- x + mult * layer_norm(y; norm_w, norm_b) (+ extra [T, W] f32, e.g. the embedding output
     re-entering before a repeated span), in place in f32, and the next sublayer's input
-    layer_norm(x; norm2_w, norm2_b) in out_dtype (norm2_w None: no next input, returns None)."""
+    layer_norm(x; norm2_w, norm2_b) in out_dtype (norm2_w None: no next input, returns None). rms: RMS
+    norms with weights only in both places (the biases are None)."""
     if not _gpu(x):
-        return ref.post_norm_add_norm(x, y, norm_w, norm_b, eps, mult, extra, norm2_w, norm2_b, out_dtype)
+        return ref.post_norm_add_norm(x, y, norm_w, norm_b, eps, mult, extra, norm2_w, norm2_b, out_dtype, rms)
     h = None if norm2_w is None else _empty(x.shape[0], x.shape[1], dtype=out_dtype, device=x.device)
-    torch.ops.bfly.post_norm_add_norm(x, y, norm_w, norm_b, float(eps), float(mult), extra, norm2_w, norm2_b, h)
+    torch.ops.bfly.post_norm_add_norm(x, y, norm_w, norm_b, float(eps), float(mult), extra, norm2_w, norm2_b, h, bool(rms))
     return h
 
 
 CONV_ACTS = {"none": 0, "silu": 1}
 
 
-def short_conv_act(z, w, state, state_slots, row_cu, positions, act: str = "silu", out_dtype=torch.float32):
-    """y_t = act(sum_j w[:, j] z_(t - taps + 1 + j)): a short causal convolution over the rows of each
+def short_conv_act(z, w, state, state_slots, row_cu, positions, act: str = "silu", out_dtype=torch.float32, bias=None):
+    """y_t = act(bias + sum_j w[:, j] z_(t - taps + 1 + j)): a short causal convolution over the rows of each
     sequence of a packed step, per channel, with an activation. z [T, C] may be a view into wider
     projected rows (any element type the model runs in); w [C, taps] f32, the last column weighs the
     current row; rows before a sequence's first row of the step come from state[slot] ([slots,
     taps - 1, C] f32, oldest first) and are zero before position 0. The state is not changed
     (short_conv_state_update_ does that, after every reader of the old state)."""
     if not _gpu(z):
-        return ref.short_conv_act(z, w, state, state_slots, row_cu, positions, act, out_dtype)
+        return ref.short_conv_act(z, w, state, state_slots, row_cu, positions, act, out_dtype, bias)
     out = _empty(z.shape[0], z.shape[1], dtype=out_dtype, device=z.device)
-    torch.ops.bfly.short_conv_act(z, w, state, state_slots, row_cu, positions, CONV_ACTS[act], out)
+    torch.ops.bfly.short_conv_act(z, w, state, state_slots, row_cu, positions, CONV_ACTS[act], out, bias)
+    return out
+
+
+def short_conv_step(z, w, state, state_slots, row_cu, positions, act: str = "silu", out_dtype=torch.float32, bias=None,
+                    one_row: bool = False):
+    """short_conv_act, then short_conv_state_update_ (nothing to update with one tap). one_row: every
+    sequence of the step has one row (decoding), both happen in one launch."""
+    taps = w.shape[1]
+    if one_row and _gpu(z):
+        out = _empty(z.shape[0], z.shape[1], dtype=out_dtype, device=z.device)
+        torch.ops.bfly.short_conv_step(z, w, bias, state if taps > 1 else None, state_slots if taps > 1 else None, positions,
+                                       CONV_ACTS[act], out)
+        return out
+    out = short_conv_act(z, w, state, state_slots, row_cu, positions, act, out_dtype, bias)
+    if taps > 1:
+        short_conv_state_update_(z, state, state_slots, row_cu, positions)
     return out
 
 
@@ -1241,3 +1274,90 @@ def delta_scan(q, k, v, b, a, a_log, dt_bias, state, state_slots, row_cu, positi
     torch.ops.bfly.delta_scan(q, k, v, b, a, a_log, dt_bias, state, state_slots, row_cu, positions, float(q_scale),
                               float(unit_eps), o)
     return o
+
+
+# ---------------------------------------------------------------------------------------
+# Pooled-block attention, linear attention with a constant decay, the selective scan
+# (csrc/kernels/pooled.hip, recur.hip)
+# ---------------------------------------------------------------------------------------
+def pool_rows(block_size: int, pool: int) -> int:
+    """Pooled rows that go with a page: the most blocks of `pool` positions that can end in one page."""
+    return (block_size + pool - 1) // pool
+
+
+def qk_norm_rows_kv(q, k, v, qn_w, kn_w, eps: float, positions, slots, k_cache, v_cache, pool=None, tables=None,
+                    row_cu=None, row_map=None, one_row: bool = False):
+    """RMS norms over a token's whole query and key projections (weights [H * D] / [G * D] f32, None: no
+    norm), a zero-padded query copy [T, H, Dp] (returned) and the paged append of k, v to K [blocks, G, BS,
+    Dp], V [blocks, G, Dvp, BS]. `pool` (P, k_pool, v_pool): then every block of P positions that a row
+    of the step completes gets its mean key and value (pool_blocks_; in the same launch when
+    `one_row`: every sequence of the step has one row)."""
+    q_out = _empty(q.shape[0], q.shape[1], k_cache.shape[3], dtype=q.dtype, device=q.device)
+    if not _gpu(q):
+        ref.qk_norm_rows_kv(q, k, v, qn_w, kn_w, eps, slots, k_cache, v_cache, q_out)
+        if pool is not None:
+            ref.pool_blocks_(k_cache, v_cache, tables, row_cu, positions, slots, *pool)
+        return q_out
+    fuse = pool is not None and one_row
+    if pool is not None and row_map is None:
+        row_map = row_seq(row_cu, q.shape[0])
+    P, kp, vp = (int(pool[0]), pool[1], pool[2]) if fuse else (0, None, None)
+    torch.ops.bfly.qk_norm_rows_kv(q, k, v, qn_w, kn_w, float(eps), slots, k_cache, v_cache, q_out, P, kp, vp,
+                                   positions if fuse else None, row_map if fuse else None, tables if fuse else None)
+    if pool is not None and not fuse:
+        torch.ops.bfly.pool_blocks(k_cache, v_cache, tables, row_map, positions, slots, int(pool[0]), pool[1], pool[2])
+    return q_out
+
+
+def pool_blocks_(k_cache, v_cache, tables, row_cu, positions, slots, pool: int, k_pool, v_pool, row_map=None):
+    """Mean key and value of every block of `pool` positions that a row of the step completes (the row's own
+    key and value are in the cache). A block's means live with the page of its last position: block b, page
+    n, pooled row b - floor(n BS / pool) of k_pool [blocks, G, pool_rows, Dp], v_pool [.., Dvp]."""
+    if not _gpu(k_cache):
+        return ref.pool_blocks_(k_cache, v_cache, tables, row_cu, positions, slots, pool, k_pool, v_pool)
+    if row_map is None:
+        row_map = row_seq(row_cu, positions.numel())
+    torch.ops.bfly.pool_blocks(k_cache, v_cache, tables, row_map, positions, slots, int(pool), k_pool, v_pool)
+
+
+DECAY_CHUNK = 64        # longest chunk of decay_scan
+
+
+def decay_powers(decay, device) -> torch.Tensor:
+    """[H, DECAY_CHUNK + 1] f32: decay[h]^i for decay_scan (powers in f64, rounded once)."""
+    d = torch.tensor(list(decay), dtype=torch.float64)
+    return torch.pow(d[:, None], torch.arange(DECAY_CHUNK + 1, dtype=torch.float64)[None]).to(torch.float32).to(device)
+
+
+def decay_scan(q, k, v, dpow, state, state_slots, row_cu, positions, act: str = "silu", one_row: bool = False):
+    """Linear attention with a constant decay per head over packed rows, S <- decay[h] S + k v^T, o = S^T q, the
+    state pooled in `state` [slots, H, D, Dv] f32 (updated in place; a sequence whose step starts at position 0
+    starts from zero). q, k [T, H, D], v [T, H, Dv] rows (views allowed), passed through `act` first; dpow =
+    decay_powers(decay). Steps of several rows per sequence run in chunks on the f32 matrix cores, steps
+    of one row (`one_row`) in place. Returns o [T, H, Dv] f32."""
+    if not _gpu(q):
+        return ref.decay_scan(q, k, v, dpow, state, state_slots, row_cu, positions, act)
+    o = _empty(q.shape[0], q.shape[1], v.shape[2], dtype=torch.float32, device=q.device)
+    torch.ops.bfly.decay_scan(q, k, v, dpow, state, state_slots, row_cu, positions, CONV_ACTS[act], bool(one_row), o)
+    return o
+
+
+def row_norm_gate(o, w, eps: float, gate, mul: float, out):
+    """out = o / sqrt(mean(o^2) + eps) * w * sigmoid(gate) * mul over whole rows: o [T, N] f32, w [N] f32, gate
+    (None: no gate) and out [T, N] rows of the model's type (views allowed)."""
+    if not _gpu(o):
+        return ref.row_norm_gate(o, w, eps, gate, mul, out)
+    torch.ops.bfly.row_norm_gate(o, w, float(eps), gate, float(mul), out)
+    return out
+
+
+def selective_scan(x, dtr, b, c, z, a_log, dt_bias, d, state, state_slots, row_cu, positions):
+    """Selective scan over packed rows with the state pooled in `state` [slots, C, N] f32 (updated in place; zero
+    at position 0): dt = softplus(dtr + dt_bias), S <- exp(-exp(a_log) dt) S + dt x B, y = S . C + d x, times silu(z).
+    x, z [T, C], b, c [T, N] rows of the model's type (views allowed), dtr [T, C] f32; a_log [C, N], dt_bias, d
+    [C] f32. Returns [T, C] in x's type."""
+    if not _gpu(x):
+        return ref.selective_scan(x, dtr, b, c, z, a_log, dt_bias, d, state, state_slots, row_cu, positions)
+    out = _empty(x.shape[0], x.shape[1], dtype=x.dtype, device=x.device)
+    torch.ops.bfly.selective_scan(x, dtr, b, c, z, a_log, dt_bias, d, state, state_slots, row_cu, positions, out)
+    return out

@@ -624,7 +624,8 @@ def rope_partial_kv(q, k, v, positions, inv_freq, slots, k_cache, v_cache):
 
 
 def attn_window_paged(q, k_cache, v_cache, tables, row_cu, positions, scale, window, keep_first, sink, out=None,
-                      out_scale=None, chunk=0, softcap=0.0, dist_bias=None, q_temp=None, maps=1, out_dtype=None):
+                      out_scale=None, chunk=0, softcap=0.0, dist_bias=None, q_temp=None, maps=1, out_dtype=None,
+                      sigmoid=False, key_bias=None, pool=None, gate=None, out_mul=1.0, dv_out=0):
     """Row r of sequence s (rows row_cu[s] .. row_cu[s+1]) at position p attends to the cached
     keys j <= p of tables[s] with p - j < window or j < keep_first; the softmax denominator
     also holds exp(sink[h]) (sink None: an ordinary softmax). out_scale [T, H] f32: every head's
@@ -635,7 +636,12 @@ def attn_window_paged(q, k_cache, v_cache, tables, row_cu, positions, scale, win
     linear form s <- s - a[h] (p - j), in that order.
     maps > 1: the key cache holds `maps` key heads per value head, and query head h reads key
     head ((h / maps) / R) * maps + h % maps (R query-head groups per value head) and its value
-    head."""
+    head.
+    Extended form (dv_out > 0; out [T, H * dv_out] rows, the first dv_out values of every head):
+    sigmoid: the weight of a visible key is sigmoid(s + key_bias[h]), not normalised over the keys;
+    pool (P, k_pool, v_pool): beside its window's tokens a row sees every block b with b P + P - 1 <= p -
+    window, with the key and value of pool_blocks_; gate [T, H * dv_out]: out *= sigmoid(gate);
+    out *= out_mul."""
     T, H, D = q.shape
     Gk, bs, Dv = k_cache.shape[1], k_cache.shape[2], v_cache.shape[2]
     G = v_cache.shape[1]
@@ -656,6 +662,14 @@ def attn_window_paged(q, k_cache, v_cache, tables, row_cu, positions, scale, win
         ok = (j <= p) & ((p - j < window) | (j < keep_first))
         if chunk > 0:
             ok = (j <= p) & ((j >= p - p % chunk) | (j < keep_first))
+        KP = VP = okp = None
+        if pool is not None:
+            P, kp, vp = pool
+            b = torch.arange((pmax - window + 1) // P if pmax - window + 1 > 0 else 0)
+            n = (b * P + P - 1) // bs
+            page, r = tables[s, n].long(), b - (n * bs) // P
+            KP, VP = kp[page, :, r].float(), vp[page, :, r].float()            # [blocks, G, D], [blocks, G, Dv]
+            okp = (b * P + P - 1)[None, :] <= p - window
         qs = q[cu[s]:cu[s + 1]].float()
         rs = torch.full_like(p, scale, dtype=torch.float32)
         if q_temp is not None:
@@ -664,21 +678,31 @@ def attn_window_paged(q, k_cache, v_cache, tables, row_cu, positions, scale, win
             gk = ((h // maps) // R) * maps + h % maps
             g = gk // maps
             sc = (qs[:, h] @ K[gk].t()) * rs
+            vals, seen = V[g], ok
+            if KP is not None:
+                sc = torch.cat([sc, (qs[:, h] @ KP[:, gk].t()) * rs], 1)
+                vals, seen = torch.cat([vals, VP[:, g]]), torch.cat([ok, okp], 1)
             if softcap > 0:
                 sc = softcap * torch.tanh(sc / softcap)
             if dist_bias is not None and dist_bias[1] is None:
                 sc = sc - dist_bias[0][h].float() * (p - j).clamp(min=0).float()
             elif dist_bias is not None:
                 sc = sc - dist_bias[0][h].float() * torch.log1p(dist_bias[1][h].float() * (p - j).clamp(min=0).float())
-            sc = sc.masked_fill(~ok, float("-inf"))
-            if sink is None:
+            sc = sc.masked_fill(~seen, float("-inf"))
+            if sigmoid:
+                w = torch.sigmoid(sc + (key_bias[h].float() if key_bias is not None else 0.0))
+            elif sink is None:
                 w = torch.softmax(sc, -1)
             else:
                 sk = sink[h].float().expand(sc.shape[0], 1)
                 w = torch.softmax(torch.cat([sc, sk], 1), -1)[:, :-1]
-            o[cu[s]:cu[s + 1], h] = w @ V[g]
+            o[cu[s]:cu[s + 1], h] = w @ vals
     if out_scale is not None:
         o = o * out_scale.float()[:, :, None]
+    if dv_out:
+        o = o[:, :, :dv_out].reshape(T, H * dv_out) * out_mul
+        if gate is not None:
+            o = o * torch.sigmoid(gate.float())
     o = o.to(out_dtype or q.dtype)
     if out is None:
         return o
@@ -737,13 +761,13 @@ def moe_route_scores(x, wr, top_k, scoring="softmax", renorm=True, bias=None, se
 
 
 def moe_glu_ffn(x, topk_ids, topk_w, gate_up_w, down_w, limit, alpha, out_dtype=None, up_offset=1.0,
-                scale_input=True, plain_act=None):
+                scale_input=True, plain_act=None, addend=None):
     """Routed GLU experts: g = min(Wg h, limit), u = clamp(Wu h, -limit, limit),
     y = g sigmoid(alpha g) (u + up_offset), output Wd y (limit inf, alpha 1, up_offset 0: the plain
     silu GLU). scale_input: the expert runs on h = w * x and a token's expert outputs are summed;
     otherwise it runs on x and the sum is weighted by w (f32). gate_up_w [E, 2F, H] (gate rows,
     then up rows), down_w [E, H, F]. plain_act "relu2": experts without a gate, y = relu(Wu h)^2
-    with gate_up_w [E, F, H]."""
+    with gate_up_w [E, F, H]. addend [T, H] (e.g. a shared expert's output) joins the f32 sum."""
     T, H = x.shape
     Fd = down_w.shape[2]
     out = torch.zeros(T, H, dtype=torch.float32, device=x.device)
@@ -764,6 +788,8 @@ def moe_glu_ffn(x, topk_ids, topk_w, gate_up_w, down_w, limit, alpha, out_dtype=
                 y = (g * torch.sigmoid(alpha * g) * (u + up_offset)).to(x.dtype).float()
             yd = y @ down_w[e].float().t()
             out[tok] += yd if scale_input else wj * yd
+    if addend is not None:
+        out = out + addend.float()
     return out.to(out_dtype or x.dtype)
 
 
@@ -1008,18 +1034,22 @@ def glu_clamp(gu, limit, alpha, up_offset, out_dtype=None, group=0):
 # sublayer, short causal convolutions with an activation on projected rows, the delta-rule
 # recurrence with pooled per-sequence state.
 # ---------------------------------------------------------------------------------------
-def post_norm_add_norm(x, y, norm_w, norm_b, eps, mult, extra, norm2_w, norm2_b, out_dtype):
+def post_norm_add_norm(x, y, norm_w, norm_b, eps, mult, extra, norm2_w, norm2_b, out_dtype, rms=False):
     """x <- x + mult * layer_norm(y; norm_w, norm_b) (+ extra), in place, f32; returns layer_norm(x;
-    norm2_w, norm2_b) in out_dtype, the next sublayer's input (norm2_w None: nothing)."""
-    v = x + mult * _layer_norm_f32(y, norm_w, norm_b, eps)
+    norm2_w, norm2_b) in out_dtype, the next sublayer's input (norm2_w None: nothing). rms: RMS norms
+    with weights only (the biases are None)."""
+    def norm(u, w, b):
+        return _rms_offset(u.float(), w, eps, 0.0) if rms else _layer_norm_f32(u, w, b, eps)
+
+    v = x + mult * norm(y, norm_w, norm_b)
     if extra is not None:
         v = v + extra.float()
     x.copy_(v)
-    return None if norm2_w is None else _layer_norm_f32(x, norm2_w, norm2_b, eps).to(out_dtype)
+    return None if norm2_w is None else norm(x, norm2_w, norm2_b).to(out_dtype)
 
 
-def short_conv_act(z, w, state, state_slots, row_cu, positions, act, out_dtype):
-    """y_t = act(sum_j w[:, j] z_(t - taps + 1 + j)) per channel over the rows of each sequence of a
+def short_conv_act(z, w, state, state_slots, row_cu, positions, act, out_dtype, bias=None):
+    """y_t = act(bias + sum_j w[:, j] z_(t - taps + 1 + j)) per channel over the rows of each sequence of a
     packed step. z [T, C] (a view of projected rows, any element type); w [C, taps] f32, the last
     column the current row's; rows before the step's first come from state[slot] ([slots, taps - 1,
     C] f32, oldest first) and are zero before position 0. act "none" | "silu". The state is not changed."""
@@ -1027,6 +1057,8 @@ def short_conv_act(z, w, state, state_slots, row_cu, positions, act, out_dtype):
     taps = w.shape[1]
     zf = z.float()
     y = torch.zeros(T, C, dtype=torch.float32, device=z.device)
+    if bias is not None:
+        y = y + bias.float()
     cu, pos = row_cu.tolist(), positions.tolist()
     sl = state_slots.tolist() if state_slots is not None else [-1] * (len(cu) - 1)
     for s in range(len(cu) - 1):
@@ -1082,3 +1114,101 @@ def delta_scan(q, k, v, b, a, a_log, dt_bias, state, state_slots, row_cu, positi
             o[t] = torch.einsum("hdv,hd->hv", S, qf[t])
         state[sl[s]] = S.transpose(1, 2)
     return o
+
+
+# ---------------------------------------------------------------------------------------
+# Pooled-block attention with norms over whole projections; linear attention with a constant
+# decay; the selective scan.
+# ---------------------------------------------------------------------------------------
+def qk_norm_rows_kv(q, k, v, qn_w, kn_w, eps, slots, k_cache, v_cache, q_out):
+    """RMS norm of a token's whole query and key projection (all heads together; weights [H * D],
+    [G * D] f32, None: no norm). q [T, H, D] -> q_out [T, H, >= D] (zero padded); k [T, G, D], v [T, G,
+    Dv] -> cache rows K [blocks, G, BS, >= D], V [blocks, G, >= Dv, BS] at slots[t] >= 0."""
+    def norm(t, w):
+        f = t.float()
+        if w is None:
+            return f
+        r = torch.rsqrt(f.flatten(1).pow(2).mean(-1) + eps)[:, None, None]
+        return f * r * w.float().view(t.shape[1], t.shape[2])
+
+    D, Dv = q.shape[2], v.shape[2]
+    q_out.zero_()
+    q_out[..., :D] = norm(q, qn_w).to(q_out.dtype)
+    kk = norm(k, kn_w)
+    bs = k_cache.shape[2]
+    ok = slots >= 0
+    sl = slots[ok].long()
+    k_cache[sl // bs, :, sl % bs, :D] = kk[ok].to(k_cache.dtype)
+    v_cache[sl // bs, :, :Dv, sl % bs] = v[ok].to(v_cache.dtype)
+    return q_out
+
+
+def pool_blocks_(k_cache, v_cache, tables, row_cu, positions, slots, pool, k_pool, v_pool):
+    """Every row whose position p completes a block of `pool` positions averages the block's cached keys
+    and values (f32 sums). Block b goes to page n = p // BS of the sequence, pooled row b - (n BS) //
+    pool of that page: k_pool [blocks, G, ceil(BS / pool), D], v_pool [.., Dv]."""
+    bs = k_cache.shape[2]
+    cu, pos, sl = row_cu.tolist(), positions.tolist(), slots.tolist()
+    for s in range(len(cu) - 1):
+        for t in range(cu[s], cu[s + 1]):
+            p = pos[t]
+            if sl[t] < 0 or (p + 1) % pool:
+                continue
+            j = torch.arange(p + 1 - pool, p + 1)
+            blk = tables[s, j // bs].long()
+            n, b = p // bs, p // pool
+            page = int(tables[s, n])
+            r = b - (n * bs) // pool
+            k_pool[page, :, r] = k_cache[blk, :, j % bs].float().mean(0).to(k_pool.dtype)
+            v_pool[page, :, r] = v_cache[blk, :, :, j % bs].float().mean(0).to(v_pool.dtype)
+
+
+def decay_scan(q, k, v, dpow, state, state_slots, row_cu, positions, act):
+    """Linear attention with a constant decay per head over packed rows, f32: q, k [T, H, D] and v [T, H,
+    Dv] first pass through silu when act == "silu"; S <- dpow[h, 1] S + k v^T, o = S^T q. The state [H, D, Dv]
+    of sequence s is read from state[state_slots[s]] unless its first row is at position 0 (then zero) and
+    written back after its last row. Returns o [T, H, Dv] f32."""
+    f = F.silu if act == "silu" else (lambda t: t)
+    qf, kf, vf = f(q.float()), f(k.float()), f(v.float())
+    T, H, D = q.shape
+    lam = dpow[:, 1].float()[:, None, None]
+    o = torch.zeros(T, H, v.shape[2], dtype=torch.float32, device=q.device)
+    cu, pos, sl = row_cu.tolist(), positions.tolist(), state_slots.tolist()
+    for s in range(len(cu) - 1):
+        if cu[s + 1] == cu[s] or sl[s] < 0:
+            continue
+        S = torch.zeros_like(state[0]) if pos[cu[s]] == 0 else state[sl[s]].clone()
+        for t in range(cu[s], cu[s + 1]):
+            S = lam * S + kf[t][:, :, None] * vf[t][:, None, :]
+            o[t] = (qf[t][:, None, :] @ S)[:, 0]
+        state[sl[s]] = S
+    return o
+
+
+def row_norm_gate(o, w, eps, gate, mul, out):
+    """out = o / sqrt(mean(o^2) + eps) * w * sigmoid(gate) * mul over whole rows [T, N]."""
+    y = _rms_offset(o.float(), w, eps, 0.0) * mul
+    if gate is not None:
+        y = y * torch.sigmoid(gate.float())
+    out.copy_(y.to(out.dtype))
+    return out
+
+
+def selective_scan(x, dtr, b, c, z, a_log, dt_bias, d, state, state_slots, row_cu, positions):
+    """Selective scan over packed rows, f32: dt = softplus(dtr + dt_bias) [T, C]; per channel and state S <-
+    exp(-exp(a_log) dt) S + dt x B, y = S . C + d x; returns y * silu(z) in x's type. x, z [T, C], b, c [T, N], state
+    [slots, C, N] (zero at position 0, written back after a sequence's last row)."""
+    A = -torch.exp(a_log.float())
+    dt = F.softplus(dtr.float() + dt_bias.float())
+    xf, bf, cf = x.float(), b.float(), c.float()
+    y = torch.zeros(x.shape, dtype=torch.float32, device=x.device)
+    cu, pos, sl = row_cu.tolist(), positions.tolist(), state_slots.tolist()
+    for s in range(len(cu) - 1):
+        if cu[s + 1] == cu[s] or sl[s] < 0:
+            continue
+        S = torch.zeros_like(state[0]) if pos[cu[s]] == 0 else state[sl[s]].clone()
+        for t in range(cu[s], cu[s + 1]):
+            S = torch.exp(dt[t][:, None] * A) * S + (dt[t] * xf[t])[:, None] * bf[t][None]
+            y[t] = S @ cf[t] + d.float() * xf[t]
+        state[sl[s]] = S
+    return (y * F.silu(z.float())).to(x.dtype)

@@ -29,15 +29,17 @@ const float* opt_f32(const optional<Tensor>& t, int64_t n, const char* what) {
   return t->data_ptr<float>();
 }
 
-void post_norm_add_norm(Tensor& x, const Tensor& y, const Tensor& nw, const Tensor& nb, double eps, double mult,
+void post_norm_add_norm(Tensor& x, const Tensor& y, const Tensor& nw, const optional<Tensor>& nb, double eps, double mult,
                         const optional<Tensor>& extra, const optional<Tensor>& nw2, const optional<Tensor>& nb2,
-                        const optional<Tensor>& h) {
-  CHK_GPU(x); CHK_GPU(y); CHK_F32(x); CHK_F32(nw); CHK_F32(nb);
+                        const optional<Tensor>& h, bool rms) {
+  CHK_GPU(x); CHK_GPU(y); CHK_F32(x); CHK_F32(nw);
   TORCH_CHECK(x.dim() == 2 && y.dim() == 2 && y.is_contiguous() && y.sizes() == x.sizes(), "post_norm_add_norm: layouts");
   const int64_t T = x.size(0), W = x.size(1);
-  TORCH_CHECK(W >= 1 && W <= kMaxRowLds && nw.numel() == W && nb.numel() == W, "post_norm_add_norm: width / norm weights");
+  TORCH_CHECK(W >= 1 && W <= kMaxRowLds && nw.numel() == W && nb.has_value() == !rms,
+              "post_norm_add_norm: width / norm weights (biases with layer norms only)");
+  const float* b1 = opt_f32(nb, W, "post_norm_add_norm: norm bias [W]");
   const float* ep = opt_f32(extra, T * W, "post_norm_add_norm: extra f32 [T, W]");
-  TORCH_CHECK(nw2.has_value() == h.has_value() && nw2.has_value() == nb2.has_value(),
+  TORCH_CHECK(nw2.has_value() == h.has_value() && nb2.has_value() == (nw2.has_value() && !rms),
               "post_norm_add_norm: the second norm needs weight, bias and an output");
   const float* w2 = opt_f32(nw2, W, "post_norm_add_norm: second norm weight [W]");
   const float* b2 = opt_f32(nb2, W, "post_norm_add_norm: second norm bias [W]");
@@ -47,8 +49,8 @@ void post_norm_add_norm(Tensor& x, const Tensor& y, const Tensor& nw, const Tens
     TORCH_CHECK(h->is_cuda() && h->is_contiguous() && h->sizes() == x.sizes(), "post_norm_add_norm: h [T, W]");
     hp = h->data_ptr();
   }
-  bfly::launch_post_norm_add_norm(x.data_ptr<float>(), y.data_ptr(), nw.data_ptr<float>(), nb.data_ptr<float>(),
-                                  (float)eps, (float)mult, ep, w2, b2, hp, (int)T, (int)W, is_f32(y), cur_stream());
+  bfly::launch_post_norm_add_norm(x.data_ptr<float>(), y.data_ptr(), nw.data_ptr<float>(), b1, (float)eps, (float)mult,
+                                  ep, w2, b2, hp, (int)T, (int)W, rms, is_f32(y), cur_stream());
 }
 
 // shared checks of a packed step's description
@@ -62,7 +64,7 @@ void check_step(const Tensor& state_slots, const Tensor& row_cu, const Tensor& p
 
 void short_conv_act(const Tensor& z, const Tensor& w, const optional<Tensor>& state,
                     const optional<Tensor>& state_slots, const Tensor& row_cu, const Tensor& positions, int64_t act,
-                    Tensor& out) {
+                    Tensor& out, const optional<Tensor>& bias) {
   CHK_GPU(z); CHK_GPU(w); CHK_F32(w); CHK_I32(row_cu); CHK_I32(positions);
   TORCH_CHECK(z.dim() == 2 && z.stride(1) == 1 && out.dim() == 2 && out.is_contiguous() && out.is_cuda() &&
                   out.sizes() == z.sizes(), "short_conv_act: z [T, C] rows, out [T, C]");
@@ -70,6 +72,7 @@ void short_conv_act(const Tensor& z, const Tensor& w, const optional<Tensor>& st
   TORCH_CHECK(w.dim() == 2 && w.size(0) == C && w.size(1) >= 1, "short_conv_act: w [C, taps]");
   const int64_t taps = w.size(1);
   TORCH_CHECK(nseq >= 0 && positions.numel() == T && (act == 0 || act == 1), "short_conv_act: row_cu / positions / act");
+  const float* bp = opt_f32(bias, C, "short_conv_act: bias f32 [C]");
   const float* sp = nullptr;
   const int* slp = nullptr;
   if (taps > 1 && state.has_value() && state_slots.has_value()) {
@@ -81,9 +84,37 @@ void short_conv_act(const Tensor& z, const Tensor& w, const optional<Tensor>& st
   }
   const bool f32 = is_f32(z), of32 = is_f32(out);
   TORCH_CHECK(of32 || !f32, "short_conv_act: f32 rows give f32 output");
-  bfly::launch_short_conv_act(z.data_ptr(), z.stride(0), w.data_ptr<float>(), sp, slp, row_cu.data_ptr<int>(), (int)nseq,
+  bfly::launch_short_conv_act(z.data_ptr(), z.stride(0), w.data_ptr<float>(), bp, sp, slp, row_cu.data_ptr<int>(), (int)nseq,
                               positions.data_ptr<int>(), out.data_ptr(), (int)T, (int)C, (int)taps, (int)act, f32, of32,
                               cur_stream());
+}
+
+// decoding: sequence s has the one row s
+void short_conv_step(const Tensor& z, const Tensor& w, const optional<Tensor>& bias, const optional<Tensor>& state,
+                     const optional<Tensor>& state_slots, const Tensor& positions, int64_t act, Tensor& out) {
+  CHK_GPU(z); CHK_GPU(w); CHK_F32(w); CHK_I32(positions);
+  TORCH_CHECK(z.dim() == 2 && z.stride(1) == 1 && out.dim() == 2 && out.is_contiguous() && out.is_cuda() &&
+                  out.sizes() == z.sizes(), "short_conv_step: z [T, C] rows, out [T, C]");
+  const int64_t T = z.size(0), C = z.size(1);
+  TORCH_CHECK(w.dim() == 2 && w.size(0) == C && w.size(1) >= 1, "short_conv_step: w [C, taps]");
+  const int64_t taps = w.size(1);
+  TORCH_CHECK(positions.is_cuda() && positions.numel() == T && (act == 0 || act == 1), "short_conv_step: positions / act");
+  const float* bp = opt_f32(bias, C, "short_conv_step: bias f32 [C]");
+  float* sp = nullptr;
+  const int* slp = nullptr;
+  if (taps > 1) {
+    TORCH_CHECK(state.has_value() && state_slots.has_value(), "short_conv_step: several taps need the history pool");
+    CHK_F32(*state); CHK_I32(*state_slots);
+    TORCH_CHECK(state->is_cuda() && state->dim() == 3 && state->size(1) == taps - 1 && state->size(2) == C &&
+                    state_slots->is_cuda() && state_slots->numel() == T,
+                "short_conv_step: state [slots, taps - 1, C] / slots [T]");
+    sp = state->data_ptr<float>();
+    slp = state_slots->data_ptr<int>();
+  }
+  const bool f32 = is_f32(z), of32 = is_f32(out);
+  TORCH_CHECK(of32 || !f32, "short_conv_step: f32 rows give f32 output");
+  bfly::launch_short_conv_step(z.data_ptr(), z.stride(0), w.data_ptr<float>(), bp, sp, slp, positions.data_ptr<int>(),
+                               out.data_ptr(), (int)T, (int)C, (int)taps, (int)act, f32, of32, cur_stream());
 }
 
 void short_conv_state_update(const Tensor& z, Tensor& state, const Tensor& state_slots, const Tensor& row_cu,
@@ -130,9 +161,11 @@ void delta_scan(const Tensor& q, const Tensor& k, const Tensor& v, const Tensor&
 }  // namespace
 
 TORCH_LIBRARY_FRAGMENT(bfly, m) {
-  m.def("post_norm_add_norm(Tensor(a!) x, Tensor y, Tensor nw, Tensor nb, float eps, float mult, Tensor? extra, "
-        "Tensor? nw2, Tensor? nb2, Tensor(b!)? h) -> ()");
+  m.def("post_norm_add_norm(Tensor(a!) x, Tensor y, Tensor nw, Tensor? nb, float eps, float mult, Tensor? extra, "
+        "Tensor? nw2, Tensor? nb2, Tensor(b!)? h, bool rms=False) -> ()");
   m.def("short_conv_act(Tensor z, Tensor w, Tensor? state, Tensor? state_slots, Tensor row_cu, Tensor positions, "
+        "int act, Tensor(a!) out, Tensor? bias=None) -> ()");
+  m.def("short_conv_step(Tensor z, Tensor w, Tensor? bias, Tensor(b!)? state, Tensor? state_slots, Tensor positions, "
         "int act, Tensor(a!) out) -> ()");
   m.def("short_conv_state_update(Tensor z, Tensor(a!) state, Tensor state_slots, Tensor row_cu, Tensor positions) -> ()");
   m.def("delta_scan(Tensor q, Tensor k, Tensor v, Tensor b, Tensor a, Tensor a_log, Tensor dt_bias, Tensor(a!) state, "
@@ -142,6 +175,7 @@ TORCH_LIBRARY_FRAGMENT(bfly, m) {
 TORCH_LIBRARY_IMPL(bfly, CUDA, m) {
   m.impl("post_norm_add_norm", &post_norm_add_norm);
   m.impl("short_conv_act", &short_conv_act);
+  m.impl("short_conv_step", &short_conv_step);
   m.impl("short_conv_state_update", &short_conv_state_update);
   m.impl("delta_scan", &delta_scan);
 }

@@ -174,7 +174,9 @@ void attn_window_paged(const Tensor& q, const Tensor& k_cache, const Tensor& v_c
                        int64_t window, int64_t keep_first, const optional<Tensor>& sink,
                        const optional<Tensor>& out_scale, bool fold_heads, const optional<Tensor>& part, Tensor& out,
                        int64_t chunk, double softcap, const optional<Tensor>& dist_a, const optional<Tensor>& dist_b,
-                       double qt_coef, int64_t qt_every, int64_t maps) {
+                       double qt_coef, int64_t qt_every, int64_t maps, bool sigmoid, const optional<Tensor>& key_bias,
+                       int64_t pool, const optional<Tensor>& k_pool, const optional<Tensor>& v_pool,
+                       const optional<Tensor>& gate, double out_mul, int64_t dv_out) {
   CHK_GPU(q); CHK_HEADS(q); CHK_SAME(k_cache, q); CHK_SAME(v_cache, q);
   bfly::AttnMod md;
   md.out_f32 = out.scalar_type() == at::kFloat && !is_f32(q);
@@ -227,8 +229,54 @@ void attn_window_paged(const Tensor& q, const Tensor& k_cache, const Tensor& v_c
     partp = part->data_ptr<float>();
     part_n = part->numel();
   }
-  TORCH_CHECK(out.is_contiguous() && out.dim() == 3 && out.size(0) == T && out.size(1) == H && out.size(2) == Dv,
-              "attn_window_paged: out");
+  if (dv_out > 0) {      // extended form: out [T, H * dv_out] rows
+    const int64_t N = H * dv_out;
+    TORCH_CHECK(out.is_cuda() && out.dim() == 2 && out.stride(1) == 1 && out.size(0) == T && out.size(1) == N && dv_out <= Dv,
+                "attn_window_paged: out [T, H * dv_out] rows");
+    TORCH_CHECK(maps == 1, "attn_window_paged: the extended form takes one map per head");
+    md.dv_out = (int)dv_out;
+    md.out_ld = out.stride(0);
+    md.out_mul = (float)out_mul;
+    bool vec = !md.out_f32 && !is_f32(q) && dv_out % 4 == 0 && out.stride(0) % 4 == 0 &&
+               reinterpret_cast<uintptr_t>(out.data_ptr()) % 8 == 0;
+    if (gate.has_value()) {
+      CHK_SAME(*gate, q);
+      TORCH_CHECK(gate->is_cuda() && gate->dim() == 2 && gate->stride(1) == 1 && gate->size(0) == T && gate->size(1) == N,
+                  "attn_window_paged: gate [T, H * dv_out] rows");
+      md.gate = gate->data_ptr();
+      md.gate_ld = gate->stride(0);
+      vec = vec && gate->stride(0) % 4 == 0 && reinterpret_cast<uintptr_t>(gate->data_ptr()) % 8 == 0;
+    }
+    md.out_vec = vec;
+    md.sigmoid = sigmoid;
+    if (key_bias.has_value()) {
+      CHK_F32(*key_bias);
+      TORCH_CHECK(sigmoid && key_bias->is_cuda() && key_bias->numel() == H, "attn_window_paged: key_bias [H] of sigmoid weights");
+      md.key_bias = key_bias->data_ptr<float>();
+    }
+    TORCH_CHECK(!(sigmoid && sink.has_value()), "attn_window_paged: a sink belongs to a softmax");
+    TORCH_CHECK(pool >= 0, "attn_window_paged: pool");
+    if (pool > 0) {
+      TORCH_CHECK(k_pool.has_value() && v_pool.has_value() && chunk == 0 && keep_first == 0 && !dist_a.has_value(),
+                  "attn_window_paged: pooled blocks need their caches and a plain sliding window");
+      CHK_SAME(*k_pool, q); CHK_SAME(*v_pool, q);
+      const int64_t pr = (bs + pool - 1) / pool;
+      TORCH_CHECK(k_pool->is_cuda() && k_pool->is_contiguous() && k_pool->dim() == 4 && k_pool->size(0) == k_cache.size(0) &&
+                      k_pool->size(1) == G && k_pool->size(2) == pr && k_pool->size(3) == D && v_pool->is_cuda() &&
+                      v_pool->is_contiguous() && v_pool->dim() == 4 && v_pool->size(0) == k_cache.size(0) &&
+                      v_pool->size(1) == G && v_pool->size(2) == pr && v_pool->size(3) == Dv,
+                  "attn_window_paged: pooled caches [blocks, G, ceil(BS / pool), D or Dv]");
+      md.pool = (int)pool;
+      md.pool_rows = (int)pr;
+      md.k_pool = k_pool->data_ptr();
+      md.v_pool = v_pool->data_ptr();
+    }
+  } else {
+    TORCH_CHECK(!sigmoid && !key_bias.has_value() && pool == 0 && !gate.has_value() && out_mul == 1.0,
+                "attn_window_paged: these options belong to the extended form (dv_out > 0)");
+    TORCH_CHECK(out.is_contiguous() && out.dim() == 3 && out.size(0) == T && out.size(1) == H && out.size(2) == Dv,
+                "attn_window_paged: out");
+  }
   TORCH_CHECK(window >= 1 && keep_first >= 0, "attn_window_paged: window >= 1, keep_first >= 0");
   if (!is_f32(q) && bfly::launch_attn_window_mfma(q.data_ptr(), q.stride(0), k_cache.data_ptr(), v_cache.data_ptr(),
                                                   tables.data_ptr<int>(), (int)tables.size(1), row_cu.data_ptr<int>(),
@@ -311,7 +359,7 @@ int64_t moe_sort_max_tiles(int64_t TK, int64_t E) { return bfly::moe_sort_max_ti
 // work: int32 [TK + (E + 1) + 2 * max_tiles + 1] = perm | offsets | tiles | ntiles
 void moe_glu_ffn(const Tensor& x, const Tensor& topk_ids, const Tensor& topk_w, const Tensor& gate_up_w,
                  const Tensor& down_w, double limit, double alpha, double up_offset, bool scale_input, Tensor& work,
-                 Tensor& hmid, Tensor& y, Tensor& out, int64_t plain_act) {
+                 Tensor& hmid, Tensor& y, Tensor& out, int64_t plain_act, const optional<Tensor>& addend) {
   CHK_GPU(x); CHK_SAME(x, gate_up_w); CHK_SAME(x, down_w); CHK_SAME(x, hmid); CHK_SAME(x, out);
   CHK_I32(topk_ids); CHK_F32(topk_w); CHK_I32(work); CHK_F32(y);
   TORCH_CHECK(x.dim() == 2 && x.stride(1) == 1 && gate_up_w.dim() == 3 && down_w.dim() == 3 &&
@@ -327,6 +375,15 @@ void moe_glu_ffn(const Tensor& x, const Tensor& topk_ids, const Tensor& topk_w, 
   TORCH_CHECK(work.numel() >= TK + E + 1 + 2 * mt + 1, "moe_glu_ffn: work buffer");
   TORCH_CHECK(hmid.is_contiguous() && hmid.numel() >= TK * F && y.numel() >= TK * Hd && out.is_contiguous() &&
                   out.size(0) == T && out.size(1) == Hd, "moe_glu_ffn: buffers");
+  const void* addp = nullptr;
+  int64_t add_ld = 0;
+  if (addend.has_value()) {
+    CHK_SAME(*addend, out);
+    TORCH_CHECK(addend->is_cuda() && addend->dim() == 2 && addend->stride(1) == 1 && addend->size(0) == T &&
+                    addend->size(1) == Hd, "moe_glu_ffn: addend [T, H] rows");
+    addp = addend->data_ptr();
+    add_ld = addend->stride(0);
+  }
   if (TK == 0) return;
   int* perm = work.data_ptr<int>();
   int* offsets = perm + TK;
@@ -343,7 +400,7 @@ void moe_glu_ffn(const Tensor& x, const Tensor& topk_ids, const Tensor& topk_w, 
   bfly::launch_moe_down(hmid.data_ptr(), perm, offsets, tiles, ntiles, (int)mt, down_w.data_ptr(), y.data_ptr<float>(),
                         (int)Hd, (int)F, f32, tr, s);
   bfly::launch_moe_sum(y.data_ptr<float>(), scale_input ? nullptr : topk_w.data_ptr<float>(), (int)K, out.data_ptr(),
-                       (int)T, (int)Hd, f32, s);
+                       (int)T, (int)Hd, f32, s, addp, (long)add_ld);
 }
 
 void sample_greedy_f32(const Tensor& logits, int64_t vstart, Tensor& out_ids, Tensor& out_scores, bool check_finite) {
@@ -374,7 +431,8 @@ TORCH_LIBRARY_FRAGMENT(bfly, m) {
   m.def("attn_window_paged(Tensor q, Tensor k_cache, Tensor v_cache, Tensor tables, Tensor row_seq, Tensor row_cu, "
         "Tensor positions, float scale, int window, int keep_first, Tensor? sink, Tensor? out_scale, bool fold_heads, "
         "Tensor(b!)? part, Tensor(a!) out, int chunk=0, float softcap=0., Tensor? dist_a=None, Tensor? dist_b=None, "
-        "float qt_coef=0., int qt_every=1, int maps=1) -> ()");
+        "float qt_coef=0., int qt_every=1, int maps=1, bool sigmoid=False, Tensor? key_bias=None, int pool=0, "
+        "Tensor? k_pool=None, Tensor? v_pool=None, Tensor? gate=None, float out_mul=1., int dv_out=0) -> ()");
   m.def("gla_scan(Tensor q, Tensor k, Tensor v, Tensor z, Tensor(a!) state, Tensor state_slots, Tensor row_cu, "
         "Tensor positions, float tau, float q_scale, Tensor(b!) o) -> ()");
   m.def("gla_out(Tensor o, Tensor g, Tensor norm_w, float eps, Tensor(a!) out) -> ()");
@@ -384,7 +442,7 @@ TORCH_LIBRARY_FRAGMENT(bfly, m) {
   m.def("moe_sort_max_tiles(int tk, int experts) -> int", &moe_sort_max_tiles);
   m.def("moe_glu_ffn(Tensor x, Tensor topk_ids, Tensor topk_w, Tensor gate_up_w, Tensor down_w, float limit, "
         "float alpha, float up_offset, bool scale_input, Tensor(a!) work, Tensor(b!) hmid, Tensor(c!) y, "
-        "Tensor(d!) out, int plain_act=0) -> ()");
+        "Tensor(d!) out, int plain_act=0, Tensor? addend=None) -> ()");
 }
 
 TORCH_LIBRARY_IMPL(bfly, CUDA, m) {

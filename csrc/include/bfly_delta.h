@@ -9,17 +9,22 @@
 
 namespace bfly {
 
-// x <- x + mult * (layer_norm(y) * nw + nb) (+ extra, nullable f32 [T, W]); h (nullable) = layer_norm(x) * nw2 + nb2
+// x <- x + mult * (layer_norm(y) * nw + nb) (+ extra, nullable f32 [T, W]); h (nullable) = layer_norm(x) * nw2 + nb2;
+// rms: RMS norms with weights only (nb, nb2 unused)
 void launch_post_norm_add_norm(float* x, const void* y, const float* nw, const float* nb, float eps, float mult,
-                               const float* extra, const float* nw2, const float* nb2, void* h, int T, int W, bool f32,
-                               hipStream_t s);
-// out[t, c] = act(sum_j w[c, j] z[t - (taps - 1 - j), c]) inside row t's sequence; rows before the step's
+                               const float* extra, const float* nw2, const float* nb2, void* h, int T, int W, bool rms,
+                               bool f32, hipStream_t s);
+// out[t, c] = act(bias[c] (nullable) + sum_j w[c, j] z[t - (taps - 1 - j), c]) inside row t's sequence; rows before the step's
 // first row of the sequence: state[slot][taps - 1 - k] is the input k steps before it, zero before
 // position 0. z rows are z_ld elements apart; state f32 [slots, taps - 1, C]; act 0 none, 1 silu;
 // out [T, C] float when out_f32 (or f32), else bf16.
-void launch_short_conv_act(const void* z, long z_ld, const float* w, const float* state, const int* state_slots,
+void launch_short_conv_act(const void* z, long z_ld, const float* w, const float* bias, const float* state, const int* state_slots,
                            const int* row_cu, int nseq, const int* positions, void* out, int T, int C, int taps, int act,
                            bool f32, bool out_f32, hipStream_t s);
+// launch_short_conv_act and the history update of a step whose sequence s has the one row s
+void launch_short_conv_step(const void* z, long z_ld, const float* w, const float* bias, float* state,
+                            const int* state_slots, const int* positions, void* out, int T, int C, int taps, int act,
+                            bool f32, bool out_f32, hipStream_t s);
 // state[slot] <- the last n rows of z of every sequence of the step (n = taps - 1; older entries shift)
 void launch_short_conv_state_update(const void* z, long z_ld, float* state, const int* state_slots, const int* row_cu,
                                     int nseq, const int* positions, int C, int n, bool f32, hipStream_t s);

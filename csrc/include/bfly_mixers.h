@@ -60,6 +60,24 @@ struct AttnMod {
   int maps = 1;                   // key heads per value head: K [blocks, G * maps, BS, D]; query heads are ordered
                                   // (head, map) and head (h, m) reads key head (g(h), m) and value head g(h)
   bool out_f32 = false;           // out is float whatever the inputs
+  // Extensions (ext()): sigmoid weights, pooled blocks, output layout. dv_out and out_ld are set whenever one
+  // of them is used.
+  bool sigmoid = false;           // weight of a visible key = sigmoid(s + key_bias[h]), no softmax
+  const float* key_bias = nullptr;  // [H]
+  int pool = 0;                   // P > 0: a row also sees block b (positions bP .. bP + P - 1) once
+                                  // bP + P - 1 <= p - window
+  int pool_rows = 0;              // pooled rows per page: k_pool [blocks, G, pool_rows, D], v_pool [.., Dv]; block b
+  const void* k_pool = nullptr;   // lives in the page n of its last position at index b - floor(n BS / P)
+  const void* v_pool = nullptr;
+  const void* gate = nullptr;     // [T, H * dv_out] rows of stride gate_ld: out *= sigmoid(gate)
+  long gate_ld = 0;
+  float out_mul = 1.f;            // out *= out_mul
+  int dv_out = 0;                 // > 0: values written per head (the cached value rows may be padded)
+  long out_ld = 0;                // row stride of out
+  bool out_vec = false;           // bf16 out / gate rows allow 8-byte accesses at every head
+  __host__ __device__ bool ext() const { return dv_out > 0; }
+  // no score modifiers
+  bool plain() const { return chunk == 0 && softcap == 0.f && !dist_a && qt_coef == 0.f && maps == 1 && !out_f32; }
 };
 
 // Row t of sequence row_seq[t] (-1: padding row, output zero) at position p sees cached keys
@@ -117,7 +135,8 @@ void launch_moe_glu_up(const void* x, long ldx, const float* topk_w, int K, cons
 // y[perm[r], :] = down_e(r) hmid[r]     (y f32, pair order)
 void launch_moe_down(const void* hmid, const int* perm, const int* offsets, const int* tiles, const int* ntiles,
                      int max_tiles, const void* down_w, float* y, int Hd, int F, bool f32, int tile_rows, hipStream_t s);
-// out[t] = sum_j wts[t * K + j] y[t * K + j]   (wts == nullptr: the plain sum)
-void launch_moe_sum(const float* y, const float* wts, int K, void* out, int T, int Hd, bool f32, hipStream_t s);
+// out[t] = sum_j wts[t * K + j] y[t * K + j] (+ add[t], rows of stride add_ld)   (wts == nullptr: the plain sum)
+void launch_moe_sum(const float* y, const float* wts, int K, void* out, int T, int Hd, bool f32, hipStream_t s,
+                    const void* add = nullptr, long add_ld = 0);
 
 }  // namespace bfly

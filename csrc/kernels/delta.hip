@@ -3,7 +3,7 @@
 //   post_norm_add_norm_kernel        x <- x + mult * layer_norm(y) (+ extra), then the next sublayer's
 //                                    input layer_norm(x) with its own weight and bias
 //   short_conv_act_kernel            y_t = act(sum_j w[:, j] z_(t - taps + 1 + j)) per channel over the
-//                                    rows of a sequence; rows before the step come from the per-sequence
+//                                    rows of a sequence (plus an optional bias); rows before the step come from the per-sequence
 //                                    history pool, zeros before position 0
 //   short_conv_state_update_kernel   the pool takes the last taps - 1 rows of every sequence
 //   delta_scan_kernel                S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q per
@@ -28,12 +28,16 @@ __device__ __forceinline__ int seq_of_row(const int* __restrict__ row_cu, int ns
   return (nseq > 0 && row_cu[lo] <= t && t < row_cu[lo + 1]) ? lo : -1;
 }
 
-// mean and 1 / sqrt(var + eps) of the row staged in LDS (f32, two passes)
+// mean and 1 / sqrt(var + eps) of the row staged in LDS (f32, two passes); RMS: 0 and 1 / sqrt(mean x^2 + eps)
+template <bool RMS>
 __device__ __forceinline__ void row_stats(const float* __restrict__ sy, int W, float eps, float* red, float& mean,
                                           float& rstd) {
-  float a = 0.f;
-  for (int c = threadIdx.x; c < W; c += blockDim.x) a += sy[c];
-  mean = block_sum(a, red) / (float)W;
+  mean = 0.f;
+  if (!RMS) {
+    float a = 0.f;
+    for (int c = threadIdx.x; c < W; c += blockDim.x) a += sy[c];
+    mean = block_sum(a, red) / (float)W;
+  }
   float q = 0.f;
   for (int c = threadIdx.x; c < W; c += blockDim.x) {
     const float d = sy[c] - mean;
@@ -44,7 +48,8 @@ __device__ __forceinline__ void row_stats(const float* __restrict__ sy, int W, f
 
 // One workgroup per row; the row of y, then the updated row of x, staged in LDS. V = 4 (W % 4 == 0):
 // 16-byte accesses (8-byte for bf16); the statistics are the same two-pass sums either way.
-template <typename T, int V>
+// RMS: RMS norms (no biases) in place of the layer norms.
+template <typename T, int V, bool RMS>
 __global__ __launch_bounds__(1024) void post_norm_add_norm_kernel(float* __restrict__ x, const T* __restrict__ y,
                                                                  const float* __restrict__ nw,
                                                                  const float* __restrict__ nb, float eps, float mult,
@@ -66,10 +71,10 @@ __global__ __launch_bounds__(1024) void post_norm_add_norm_kernel(float* __restr
   }
   __syncthreads();
   float mean, rstd;
-  row_stats(sy, W, eps, red, mean, rstd);
+  row_stats<RMS>(sy, W, eps, red, mean, rstd);
   for (int c = V * threadIdx.x; c < W; c += V * blockDim.x) {
     const fv yv = *reinterpret_cast<const fv*>(sy + c), wv = *reinterpret_cast<const fv*>(nw + c),
-             bv = *reinterpret_cast<const fv*>(nb + c);
+             bv = RMS ? fv(0.f) : *reinterpret_cast<const fv*>(nb + c);
     fv v = *reinterpret_cast<const fv*>(x + t * W + c);
 #pragma unroll
     for (int e = 0; e < V; ++e) v[e] = v[e] + mult * ((yv[e] - mean) * rstd * wv[e] + bv[e]);
@@ -83,10 +88,10 @@ __global__ __launch_bounds__(1024) void post_norm_add_norm_kernel(float* __restr
   }
   if (!h) return;
   __syncthreads();
-  row_stats(sy, W, eps, red, mean, rstd);
+  row_stats<RMS>(sy, W, eps, red, mean, rstd);
   for (int c = V * threadIdx.x; c < W; c += V * blockDim.x) {
     const fv xv = *reinterpret_cast<const fv*>(sy + c), wv = *reinterpret_cast<const fv*>(nw2 + c),
-             bv = *reinterpret_cast<const fv*>(nb2 + c);
+             bv = RMS ? fv(0.f) : *reinterpret_cast<const fv*>(nb2 + c);
     tv o;
 #pragma unroll
     for (int e = 0; e < V; ++e) o[e] = (T)((xv[e] - mean) * rstd * wv[e] + bv[e]);
@@ -94,10 +99,11 @@ __global__ __launch_bounds__(1024) void post_norm_add_norm_kernel(float* __restr
   }
 }
 
-// one thread per (row, channel); the taps are summed oldest first
+// one thread per (row, channel); the bias (nullable), then the taps oldest first
 template <typename TI, typename TO>
 __global__ __launch_bounds__(256) void short_conv_act_kernel(const TI* __restrict__ z, long z_ld,
                                                              const float* __restrict__ w,
+                                                             const float* __restrict__ bias,
                                                              const float* __restrict__ state,
                                                              const int* __restrict__ state_slots,
                                                              const int* __restrict__ row_cu, int nseq,
@@ -107,7 +113,7 @@ __global__ __launch_bounds__(256) void short_conv_act_kernel(const TI* __restric
   const int c = blockIdx.y * blockDim.x + threadIdx.x;
   if (c >= C) return;
   const int s = seq_of_row(row_cu, nseq, t);
-  float acc = 0.f;
+  float acc = bias ? bias[c] : 0.f;
   if (s >= 0) {
     const int a = row_cu[s], p = positions[t];
     const int slot = state_slots ? state_slots[s] : -1;
@@ -131,6 +137,7 @@ __global__ __launch_bounds__(256) void short_conv_act_kernel(const TI* __restric
 template <typename TI, typename TO>
 __global__ __launch_bounds__(256) void short_conv_act_rows_kernel(const TI* __restrict__ z, long z_ld,
                                                                   const float* __restrict__ w,
+                                                                  const float* __restrict__ bias,
                                                                   const float* __restrict__ state,
                                                                   const int* __restrict__ state_slots,
                                                                   const int* __restrict__ row_cu, int nseq,
@@ -149,6 +156,7 @@ __global__ __launch_bounds__(256) void short_conv_act_rows_kernel(const TI* __re
   for (int j = 0; j <= MAXN; ++j)
 #pragma unroll
     for (int e = 0; e < 4; ++e) wv[j][e] = j < taps ? w[(long)(c + e) * taps + j] : 0.f;
+  const f32x4 bv = bias ? *reinterpret_cast<const f32x4*>(bias + c) : f32x4{0.f, 0.f, 0.f, 0.f};
   auto ld = [&](long row) {
     const tiv v = *reinterpret_cast<const tiv*>(z + row * z_ld + c);
     return f32x4{(float)v[0], (float)v[1], (float)v[2], (float)v[3]};
@@ -161,7 +169,7 @@ __global__ __launch_bounds__(256) void short_conv_act_rows_kernel(const TI* __re
       send = s >= 0 ? row_cu[s + 1] : t + 1;
       fetch = true;
     }
-    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+    f32x4 acc = bv;
     if (s >= 0) {
       const f32x4 zc = ld(t);
       if (fetch) {
@@ -202,6 +210,33 @@ __global__ __launch_bounds__(256) void short_conv_act_rows_kernel(const TI* __re
     for (int e = 0; e < 4; ++e) o[e] = (TO)(act == 1 ? acc[e] / (1.f + expf(-acc[e])) : acc[e]);
     *reinterpret_cast<tov*>(out + (long)t * C + c) = o;
   }
+}
+
+// Decoding: every sequence has one row (row s), so the convolution and its history update share a launch
+// and a thread. Same order of summation as above.
+template <typename TI, typename TO>
+__global__ __launch_bounds__(256) void short_conv_step_kernel(const TI* __restrict__ z, long z_ld,
+                                                              const float* __restrict__ w,
+                                                              const float* __restrict__ bias, float* __restrict__ state,
+                                                              const int* __restrict__ state_slots,
+                                                              const int* __restrict__ positions, TO* __restrict__ out,
+                                                              int C, int taps, int act) {
+  const long s = blockIdx.x;
+  const int c = blockIdx.y * blockDim.x + threadIdx.x;
+  if (c >= C) return;
+  const int p = positions[s], slot = state_slots ? state_slots[s] : -1, n = taps - 1;
+  const float zc = (float)z[s * z_ld + c];
+  float* S = state + (long)slot * n * C + c;
+  float acc = bias ? bias[c] : 0.f;
+  for (int j = 0; j < n; ++j) {
+    const float v = (slot >= 0 && p - (n - j) >= 0) ? S[(long)j * C] : 0.f;
+    acc = fmaf(w[(long)c * taps + j], v, acc);
+    if (slot >= 0 && j > 0) S[(long)(j - 1) * C] = v;       // (entry j - 1 was read one iteration ago)
+  }
+  acc = fmaf(w[(long)c * taps + n], zc, acc);
+  if (slot >= 0 && n > 0) S[(long)(n - 1) * C] = zc;
+  if (act == 1) acc = acc / (1.f + expf(-acc));
+  out[s * C + c] = (TO)acc;
 }
 
 // one thread per (sequence, channel): entry i of the new history is old entry i + len while that
@@ -412,19 +447,38 @@ int row_threads(int W) { return std::min(1024, std::max(64, (W / 4 + 63) / 64 * 
 }  // namespace
 
 void launch_post_norm_add_norm(float* x, const void* y, const float* nw, const float* nb, float eps, float mult,
-                               const float* extra, const float* nw2, const float* nb2, void* h, int T, int W, bool f32,
-                               hipStream_t s) {
+                               const float* extra, const float* nw2, const float* nb2, void* h, int T, int W, bool rms,
+                               bool f32, hipStream_t s) {
   if (T <= 0) return;
   const size_t sm = (size_t)W * sizeof(float);
-#define BFLY_PNAN(TT, V)                                                                                          \
-  post_norm_add_norm_kernel<TT, V><<<T, row_threads(W), sm, s>>>(x, (const TT*)y, nw, nb, eps, mult, extra, nw2, nb2, \
-                                                                 (TT*)h, W)
-  if (W % 4 == 0) { if (f32) BFLY_PNAN(float, 4); else BFLY_PNAN(bf16, 4); }
-  else { if (f32) BFLY_PNAN(float, 1); else BFLY_PNAN(bf16, 1); }
+#define BFLY_PNAN(TT, V, R)                                                                                          \
+  post_norm_add_norm_kernel<TT, V, R><<<T, row_threads(W), sm, s>>>(x, (const TT*)y, nw, nb, eps, mult, extra, nw2, nb2, \
+                                                                    (TT*)h, W)
+#define BFLY_PNAN2(TT, V)        \
+  {                              \
+    if (rms) BFLY_PNAN(TT, V, true); else BFLY_PNAN(TT, V, false); \
+  }
+  if (W % 4 == 0) { if (f32) BFLY_PNAN2(float, 4) else BFLY_PNAN2(bf16, 4) }
+  else { if (f32) BFLY_PNAN2(float, 1) else BFLY_PNAN2(bf16, 1) }
+#undef BFLY_PNAN2
 #undef BFLY_PNAN
 }
 
-void launch_short_conv_act(const void* z, long z_ld, const float* w, const float* state, const int* state_slots,
+void launch_short_conv_step(const void* z, long z_ld, const float* w, const float* bias, float* state,
+                            const int* state_slots, const int* positions, void* out, int T, int C, int taps, int act,
+                            bool f32, bool out_f32, hipStream_t s) {
+  if (T <= 0 || C <= 0) return;
+  dim3 grid(T, (C + 255) / 256);
+#define BFLY_SCS(TI, TO)                                                                                              \
+  short_conv_step_kernel<TI, TO><<<grid, 256, 0, s>>>((const TI*)z, z_ld, w, bias, state, state_slots, positions, (TO*)out, \
+                                                      C, taps, act)
+  if (f32) BFLY_SCS(float, float);
+  else if (out_f32) BFLY_SCS(bf16, float);
+  else BFLY_SCS(bf16, bf16);
+#undef BFLY_SCS
+}
+
+void launch_short_conv_act(const void* z, long z_ld, const float* w, const float* bias, const float* state, const int* state_slots,
                            const int* row_cu, int nseq, const int* positions, void* out, int T, int C, int taps, int act,
                            bool f32, bool out_f32, hipStream_t s) {
   if (T <= 0 || C <= 0) return;
@@ -434,7 +488,7 @@ void launch_short_conv_act(const void* z, long z_ld, const float* w, const float
     const int RB = std::min(16, std::max(1, T / 512));
     dim3 g2((T + RB - 1) / RB, (C / 4 + 255) / 256);
 #define BFLY_SCR(TI, TO)                                                                                             \
-  short_conv_act_rows_kernel<TI, TO><<<g2, 256, 0, s>>>((const TI*)z, z_ld, w, state, state_slots, row_cu, nseq,     \
+  short_conv_act_rows_kernel<TI, TO><<<g2, 256, 0, s>>>((const TI*)z, z_ld, w, bias, state, state_slots, row_cu, nseq,     \
                                                         positions, (TO*)out, C, taps, act, T, RB)
     if (f32) BFLY_SCR(float, float);
     else if (out_f32) BFLY_SCR(bf16, float);
@@ -444,7 +498,7 @@ void launch_short_conv_act(const void* z, long z_ld, const float* w, const float
   }
   dim3 grid(T, (C + 255) / 256);
 #define BFLY_SC(TI, TO)                                                                                              \
-  short_conv_act_kernel<TI, TO><<<grid, 256, 0, s>>>((const TI*)z, z_ld, w, state, state_slots, row_cu, nseq, positions, \
+  short_conv_act_kernel<TI, TO><<<grid, 256, 0, s>>>((const TI*)z, z_ld, w, bias, state, state_slots, row_cu, nseq, positions, \
                                                      (TO*)out, C, taps, act)
   if (f32) BFLY_SC(float, float);
   else if (out_f32) BFLY_SC(bf16, float);

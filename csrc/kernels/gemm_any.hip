@@ -225,7 +225,7 @@ __global__ __launch_bounds__(256) void moe_down_kernel(const T* __restrict__ hmi
 
 template <typename T>
 __global__ void moe_sum_kernel(const float* __restrict__ y, const float* __restrict__ wts, int Kc, T* __restrict__ out,
-                               long T_, int Hd) {
+                               long T_, int Hd, const T* __restrict__ add, long add_ld) {
   const long n = T_ * Hd;
   for (long i = blockIdx.x * (long)blockDim.x + threadIdx.x; i < n; i += (long)gridDim.x * blockDim.x) {
     const long t = i / Hd;
@@ -236,7 +236,35 @@ __global__ void moe_sum_kernel(const float* __restrict__ y, const float* __restr
     } else {
       for (int j = 0; j < Kc; ++j) s += y[(t * Kc + j) * Hd + c];
     }
+    if (add) s += (float)add[t * add_ld + c];
     out[i] = (T)s;
+  }
+}
+
+// The same sum, four columns per thread (Hd % 4 == 0, 8 / 16-byte aligned rows of `add`).
+template <typename T>
+__global__ __launch_bounds__(256) void moe_sum4_kernel(const float* __restrict__ y, const float* __restrict__ wts, int Kc,
+                                                       T* __restrict__ out, int Hd, const T* __restrict__ add,
+                                                       long add_ld) {
+  typedef T tv __attribute__((ext_vector_type(4)));
+  const long t = blockIdx.x;
+  for (int c = 4 * threadIdx.x; c < Hd; c += 4 * blockDim.x) {
+    f32x4 s = {0.f, 0.f, 0.f, 0.f};
+    for (int j = 0; j < Kc; ++j) {
+      const f32x4 v = *reinterpret_cast<const f32x4*>(y + (t * Kc + j) * Hd + c);
+      const float w = wts ? wts[t * Kc + j] : 1.f;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) s[e] = fmaf(w, v[e], s[e]);
+    }
+    if (add) {
+      const tv a = *reinterpret_cast<const tv*>(add + t * add_ld + c);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) s[e] += (float)a[e];
+    }
+    tv o;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) o[e] = (T)s[e];
+    *reinterpret_cast<tv*>(out + t * Hd + c) = o;
   }
 }
 
@@ -712,11 +740,19 @@ void launch_moe_down(const void* hmid, const int* perm, const int* offsets, cons
                                               Hd, F);
 }
 
-void launch_moe_sum(const float* y, const float* wts, int K, void* out, int T, int Hd, bool f32, hipStream_t s) {
+void launch_moe_sum(const float* y, const float* wts, int K, void* out, int T, int Hd, bool f32, hipStream_t s,
+                    const void* add, long add_ld) {
   const long n = (long)T * Hd;
   if (n <= 0) return;
-  if (f32) moe_sum_kernel<float><<<ew_blocks(n), 256, 0, s>>>(y, wts, K, (float*)out, T, Hd);
-  else moe_sum_kernel<bf16><<<ew_blocks(n), 256, 0, s>>>(y, wts, K, (bf16*)out, T, Hd);
+  const size_t al = f32 ? 16 : 8;
+  if (Hd % 4 == 0 && reinterpret_cast<uintptr_t>(out) % al == 0 && reinterpret_cast<uintptr_t>(y) % 16 == 0 &&
+      (!add || (add_ld % 4 == 0 && reinterpret_cast<uintptr_t>(add) % al == 0))) {
+    if (f32) moe_sum4_kernel<float><<<T, 256, 0, s>>>(y, wts, K, (float*)out, Hd, (const float*)add, add_ld);
+    else moe_sum4_kernel<bf16><<<T, 256, 0, s>>>(y, wts, K, (bf16*)out, Hd, (const bf16*)add, add_ld);
+    return;
+  }
+  if (f32) moe_sum_kernel<float><<<ew_blocks(n), 256, 0, s>>>(y, wts, K, (float*)out, T, Hd, (const float*)add, add_ld);
+  else moe_sum_kernel<bf16><<<ew_blocks(n), 256, 0, s>>>(y, wts, K, (bf16*)out, T, Hd, (const bf16*)add, add_ld);
 }
 
 }  // namespace bfly
