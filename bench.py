@@ -92,14 +92,17 @@ def build_parser() -> argparse.ArgumentParser:
                     help="single-stage layouts: host waits for each step's tokens before scheduling the "
                          "next (default: EngineConfig.async_decode, the next step overlaps the host work)")
     ap.add_argument("--out", default=None, help="also write the JSON line here")
-    ap.add_argument("--mixer-family", default="nesizen", choices=["nesizen", "zinesun", "lizizen", "gevipel"],
+    ap.add_argument("--mixer-family", default="nesizen", choices=["nesizen", "zinesun", "lizizen", "gevipel", "vuladra"],
                     help="with --mixer-compare: the heterogeneous family that is timed (nesizen: beside a Mixtral "
                          "stack; zinesun: latent attention beside a Nesizen stack of plain windowed attention; "
                          "lizizen: parallel layers of distance-biased and differential attention with dense GLU "
                          "feed-forwards beside a Nesizen stack of plain attention with dense feed-forwards; "
                          "gevipel: sandwich-normed layers of sloped window attention, the gated delta rule and latent "
                          "attention with a sink over routed plain experts beside a Nesizen stack of windowed "
-                         "attention and gated linear attention over routed GLU experts)")
+                         "attention and gated linear attention over routed GLU experts; "
+                         "vuladra: windowed attention beside decayed linear attention, the selective scan and sigmoid "
+                         "attention with pooled blocks over dense and routed GLUs with a shared expert beside a Nesizen "
+                         "stack of windowed attention and gated linear attention)")
     ap.add_argument("--mixer-compare", default=None, metavar="SIZES",
                     help="instead of the headline run: prefill and decode throughput of a Nesizen stack "
                          "(windowed attention, shared keys, gated linear attention, sigmoid MoE) beside a "
@@ -251,6 +254,36 @@ def run_mixer_compare(a) -> int:
                                                   "mlp": moe},
                                                  {"type": "gla", "mixer": gla, "mlp": moe}]}, name=f"nesizen-mix-{size}")
             pair = (gev, nes4)
+        if a.mixer_family == "vuladra":
+            # windowed attention beside decayed linear attention (half the heads each), the selective scan with
+            # twice the width, 16 states and 4 taps, and sigmoid attention over a window and pooled blocks of 16
+            # tokens; one dense silu GLU (two thirds of the width: the parameters of the counterpart's two matrices),
+            # routed clamped GLUs with a shared expert (one routed choice less: the same active FLOPs); beside
+            # windowed GQA attention and gated linear attention of the same heads and window, one stream
+            w2 = win // 2
+            side = {"left": {"heads": H // 2, "kv_heads": max(G // 2, 1), "dim": D, "vdim": D, "scale": D ** -0.5,
+                             "mask": {"size": w2}}, "left_scale": 1.0, "right_scale": 0.8,
+                    "right": {"heads": H // 2, "dim": D, "vdim": D,
+                              "decay": [1.0 - 2.0 ** (-3 - 5 * i / (H // 2)) for i in range(H // 2)]}}
+            mam = {"inner": 2 * W, "state": 16, "dt_rank": W // 16, "conv": 4}
+            pol = {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "scale": D ** -0.5, "mask": {"size": w2, "pool": 16}}
+            vmoe = {"kind": "moe", "expert": {"ff": eff, "limit": 7.0}, "router": {"experts": E, "top": top - 1},
+                    "shared": {"ff": eff, "limit": 7.0}}
+            vul = ModelConfig.from_vuladra({"architecture": "Vuladra", "vocab": 32000, "width": W, "norm": {"eps": 1e-6},
+                                            "layers": [
+                                                {"type": "parallel", "mixer": side,
+                                                 "mlp": {"kind": "dense", "ff": 2 * dff // 3 // 128 * 128}},
+                                                {"type": "mamba1", "mixer": mam, "mlp": vmoe},
+                                                {"type": "attention", "mixer": pol, "mlp": vmoe},
+                                                {"type": "mamba1", "mixer": mam, "mlp": vmoe}]}, name=f"vuladra-{size}")
+            plain = dict(attn, mask={"size": w2, "keep_first": 0})
+            nes5 = ModelConfig.from_nesizen({"architecture": "Nesizen", "vocab": 32000, "width": W, "streams": 1,
+                                             "norm": {"eps": 1e-6}, "layers": [
+                                                 {"type": "attention", "mixer": plain, "mlp": {"kind": "dense", "ff": dff}},
+                                                 {"type": "gla", "mixer": gla, "mlp": moe},
+                                                 {"type": "attention", "mixer": plain, "mlp": moe},
+                                                 {"type": "gla", "mixer": gla, "mlp": moe}]}, name=f"nesizen-scan-{size}")
+            pair = (vul, nes5)
         for cfg in pair:
             ecfg = EngineConfig(max_batch=B, max_seq_len=P + K + Wm + 8, max_prefill_tokens=8192,
                                 kv_cache_tokens=B * (P + K + Wm + 40), use_graphs=not a.no_graphs,

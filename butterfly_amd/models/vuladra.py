@@ -396,9 +396,9 @@ class VuladraLM(PackedStack):
         x = ops.short_conv_step(u[:, :C], p[pre + "conv"], self.state[si], meta["state_slots"], meta["row_cu"], fb.positions,
                                 "silu", self.dtype, p[pre + "conv.b"], meta["one_row"])
         s = ops.linear_act(x, p[pre + "x"])                                     # dt | B | C
-        dt = ops.linear_act(s[:, :R], p[pre + "dt"], out_dtype=torch.float32)
-        y = ops.selective_scan(x, dt, s[:, R:R + N], s[:, R + N:R + 2 * N], u[:, C:2 * C], p[pre + "A_log"], p[pre + "dt.b"],
-                               p[pre + "D"], self.state[si + 1], meta["state_slots"], meta["row_cu"], fb.positions)
+        y = ops.selective_scan(x, s[:, :R], p[pre + "dt"], s[:, R:R + N], s[:, R + N:R + 2 * N], u[:, C:2 * C],
+                               p[pre + "A_log"], p[pre + "dt.b"], p[pre + "D"], self.state[si + 1], meta["state_slots"],
+                               meta["row_cu"], fb.positions, meta["one_row"])
         return ops.linear_act(y, p[pre + "o"])
 
     def _glu(self, name, h, ff, limit, alpha, offset):

@@ -1351,11 +1351,17 @@ def row_norm_gate(o, w, eps: float, gate, mul: float, out):
     return out
 
 
-def selective_scan(x, dtr, b, c, z, a_log, dt_bias, d, state, state_slots, row_cu, positions):
+def selective_scan(x, low, w_dt, b, c, z, a_log, dt_bias, d, state, state_slots, row_cu, positions, one_row: bool = False):
     """Selective scan over packed rows with the state pooled in `state` [slots, C, N] f32 (updated in place; zero
-    at position 0): dt = softplus(dtr + dt_bias), S <- exp(-exp(a_log) dt) S + dt x B, y = S . C + d x, times silu(z).
-    x, z [T, C], b, c [T, N] rows of the model's type (views allowed), dtr [T, C] f32; a_log [C, N], dt_bias, d
-    [C] f32. Returns [T, C] in x's type."""
+    at position 0): dt = softplus(w_dt low + dt_bias), S <- exp(-exp(a_log) dt) S + dt x B, y = S . C + d x, times silu(z).
+    x, z [T, C], low [T, R], b, c [T, N] rows of the model's type (views allowed), w_dt [C, R]; a_log [C, N],
+    dt_bias, d [C] f32. Returns [T, C] in x's type. The low-rank projection keeps its f32 accumulator; with
+    `one_row` (every sequence of the step has one row) it happens inside the step's one launch."""
+    if one_row and _gpu(x):
+        out = _empty(x.shape[0], x.shape[1], dtype=x.dtype, device=x.device)
+        torch.ops.bfly.selective_step(x, low, w_dt, b, c, z, a_log, dt_bias, d, state, state_slots, positions, out)
+        return out
+    dtr = linear_act(low, w_dt, out_dtype=torch.float32)
     if not _gpu(x):
         return ref.selective_scan(x, dtr, b, c, z, a_log, dt_bias, d, state, state_slots, row_cu, positions)
     out = _empty(x.shape[0], x.shape[1], dtype=x.dtype, device=x.device)

@@ -76,20 +76,44 @@ void row_norm_gate(const Tensor& o, const Tensor& w, double eps, const optional<
                              out.stride(0), (int)o.size(0), (int)o.size(1), is_f32(out), cur_stream());
 }
 
-void selective_scan(const Tensor& x, const Tensor& dtr, const Tensor& b, const Tensor& c, const Tensor& z,
-                    const Tensor& a_log, const Tensor& dt_bias, const Tensor& d, Tensor& state, const Tensor& state_slots,
-                    const Tensor& row_cu, const Tensor& positions, Tensor& out) {
-  CHK_ROWS(x); CHK_ROWS(dtr); CHK_ROWS(b); CHK_ROWS(c); CHK_ROWS(z); CHK_ROWS(out);
+// checks shared by the scan and the step: x, z [T, C], B, C [T, N] rows, a_log [C, N], state [slots, C, N]
+void check_selective(const Tensor& x, const Tensor& b, const Tensor& c, const Tensor& z, const Tensor& a_log,
+                     const Tensor& dt_bias, const Tensor& d, const Tensor& state, const Tensor& out) {
+  CHK_ROWS(x); CHK_ROWS(b); CHK_ROWS(c); CHK_ROWS(z); CHK_ROWS(out);
   CHK_SAME(b, x); CHK_SAME(c, x); CHK_SAME(z, x); CHK_SAME(out, x);
   CHK_F32(a_log); CHK_F32(dt_bias); CHK_F32(d); CHK_F32(state);
   const int64_t T = x.size(0), C = x.size(1), N = a_log.size(1);
-  TORCH_CHECK(dtr.scalar_type() == at::kFloat && dtr.size(0) == T && dtr.size(1) == C && z.sizes() == x.sizes(),
-              "selective_scan: x, z [T, C], dtr f32 [T, C]");
-  TORCH_CHECK(a_log.dim() == 2 && a_log.size(0) == C && dt_bias.numel() == C && d.numel() == C,
-              "selective_scan: a_log [C, N], dt_bias, d [C]");
-  TORCH_CHECK(b.size(0) == T && b.size(1) == N && c.sizes() == b.sizes(), "selective_scan: B, C [T, N]");
-  TORCH_CHECK(state.dim() == 3 && state.size(1) == C && state.size(2) == N, "selective_scan: state [slots, C, N]");
-  TORCH_CHECK(out.is_contiguous() && out.sizes() == x.sizes(), "selective_scan: out [T, C]");
+  TORCH_CHECK(a_log.dim() == 2 && a_log.size(0) == C && dt_bias.numel() == C && d.numel() == C && z.sizes() == x.sizes(),
+              "selective scan: x, z [T, C], a_log [C, N], dt_bias, d [C]");
+  TORCH_CHECK(b.size(0) == T && b.size(1) == N && c.sizes() == b.sizes(), "selective scan: B, C [T, N]");
+  TORCH_CHECK(state.dim() == 3 && state.size(1) == C && state.size(2) == N, "selective scan: state [slots, C, N]");
+  TORCH_CHECK(out.is_contiguous() && out.sizes() == x.sizes(), "selective scan: out [T, C]");
+}
+
+void selective_step(const Tensor& x, const Tensor& low, const Tensor& wdt, const Tensor& b, const Tensor& c, const Tensor& z,
+                    const Tensor& a_log, const Tensor& dt_bias, const Tensor& d, Tensor& state, const Tensor& state_slots,
+                    const Tensor& positions, Tensor& out) {
+  check_selective(x, b, c, z, a_log, dt_bias, d, state, out);
+  CHK_ROWS(low); CHK_SAME(low, x); CHK_SAME(wdt, x); CHK_I32(state_slots); CHK_I32(positions);
+  const int64_t T = x.size(0), C = x.size(1), N = a_log.size(1), R = low.size(1);
+  TORCH_CHECK(low.size(0) == T && wdt.is_cuda() && wdt.is_contiguous() && wdt.dim() == 2 && wdt.size(0) == C &&
+                  wdt.size(1) == R && R <= 8192, "selective_step: low [T, R], wdt [C, R]");
+  TORCH_CHECK(state_slots.numel() == T && positions.numel() == T, "selective_step: one row per sequence");
+  const int rc = bfly::launch_selective_step(
+      x.data_ptr(), x.stride(0), low.data_ptr(), low.stride(0), wdt.data_ptr(), (int)R, b.data_ptr(), b.stride(0),
+      c.data_ptr(), c.stride(0), z.data_ptr(), z.stride(0), a_log.data_ptr<float>(), dt_bias.data_ptr<float>(),
+      d.data_ptr<float>(), state.data_ptr<float>(), state_slots.data_ptr<int>(), positions.data_ptr<int>(), out.data_ptr(),
+      (int)T, (int)C, (int)N, is_f32(x), cur_stream());
+  TORCH_CHECK(rc == 0, "selective_step: ", N, " states per channel are not supported (<= 256)");
+}
+
+void selective_scan(const Tensor& x, const Tensor& dtr, const Tensor& b, const Tensor& c, const Tensor& z,
+                    const Tensor& a_log, const Tensor& dt_bias, const Tensor& d, Tensor& state, const Tensor& state_slots,
+                    const Tensor& row_cu, const Tensor& positions, Tensor& out) {
+  check_selective(x, b, c, z, a_log, dt_bias, d, state, out);
+  CHK_ROWS(dtr);
+  const int64_t T = x.size(0), C = x.size(1), N = a_log.size(1);
+  TORCH_CHECK(dtr.scalar_type() == at::kFloat && dtr.size(0) == T && dtr.size(1) == C, "selective_scan: dtr f32 [T, C]");
   check_step(state_slots, row_cu, positions, T, "selective_scan");
   const int rc = bfly::launch_selective_scan(
       x.data_ptr(), x.stride(0), dtr.data_ptr<float>(), dtr.stride(0), b.data_ptr(), b.stride(0), c.data_ptr(), c.stride(0),
@@ -174,6 +198,8 @@ TORCH_LIBRARY_FRAGMENT(bfly, m) {
   m.def("row_norm_gate(Tensor o, Tensor w, float eps, Tensor? gate, float mul, Tensor(a!) out) -> ()");
   m.def("selective_scan(Tensor x, Tensor dtr, Tensor b, Tensor c, Tensor z, Tensor a_log, Tensor dt_bias, Tensor d, "
         "Tensor(a!) state, Tensor state_slots, Tensor row_cu, Tensor positions, Tensor(b!) out) -> ()");
+  m.def("selective_step(Tensor x, Tensor low, Tensor wdt, Tensor b, Tensor c, Tensor z, Tensor a_log, Tensor dt_bias, "
+        "Tensor d, Tensor(a!) state, Tensor state_slots, Tensor positions, Tensor(b!) out) -> ()");
   m.def("qk_norm_rows_kv(Tensor q, Tensor k, Tensor v, Tensor? qw, Tensor? kw, float eps, Tensor slots, "
         "Tensor(a!) k_cache, Tensor(b!) v_cache, Tensor(c!) q_out, int pool, Tensor(d!)? k_pool, Tensor(e!)? v_pool, "
         "Tensor? positions, Tensor? row_seq, Tensor? tables) -> ()");
@@ -185,6 +211,7 @@ TORCH_LIBRARY_IMPL(bfly, CUDA, m) {
   m.impl("decay_scan", &decay_scan);
   m.impl("row_norm_gate", &row_norm_gate);
   m.impl("selective_scan", &selective_scan);
+  m.impl("selective_step", &selective_step);
   m.impl("qk_norm_rows_kv", &qk_norm_rows_kv);
   m.impl("pool_blocks", &pool_blocks);
 }

@@ -29,6 +29,12 @@ int launch_selective_scan(const void* x, long x_ld, const float* dtr, long dt_ld
                           float* state, const int* state_slots, const int* row_cu, int nseq, const int* positions,
                           void* out, int T, int C, int N, bool f32, hipStream_t s);
 
+// launch_selective_scan for a step whose sequence s has the one row s, with dtr = wdt low: low [T, R] rows, wdt [C, R]
+int launch_selective_step(const void* x, long x_ld, const void* low, long l_ld, const void* wdt, int R, const void* b,
+                          long b_ld, const void* c, long c_ld, const void* z, long z_ld, const float* a_log,
+                          const float* dt_bias, const float* d, float* state, const int* state_slots, const int* positions,
+                          void* out, int T, int C, int N, bool f32, hipStream_t s);
+
 // RMS norm of a token's whole query row [H * D] and key row [G * D] (weights qw, kw of those sizes; nullptr: no
 // norm), the queries copied to q_out [T, H, Dp] (zero padded), keys and values appended to K [blocks, G, BS, Dp],
 // V [blocks, G, Dvp, BS] at slots[t] >= 0. pool > 0 (only for steps in which every row is a sequence of its

@@ -34,13 +34,19 @@ __device__ __forceinline__ void pool_block(const T* k_cache, const T* v_cache, i
   for (int j = 0; j < P;) {
     const long blk = tab[page];
     const int run = min(P - j, bs - off);
-    if (i < Dp) {
-      const T* kr = k_cache + ((blk * G + g) * bs + off) * Dp + i;
-      for (int u = 0; u < run; ++u) a += (float)kr[(long)u * Dp];
-    } else {
-      const T* vr = v_cache + ((blk * G + g) * Dvp + (i - Dp)) * bs + off;
-      for (int u = 0; u < run; ++u) a += (float)vr[u];
+    // (eight loads in flight; the sum stays in ascending order)
+    const bool key = i < Dp;
+    const T* src = key ? k_cache + ((blk * G + g) * bs + off) * Dp + i : v_cache + ((blk * G + g) * Dvp + (i - Dp)) * bs + off;
+    const long step = key ? Dp : 1;
+    int u = 0;
+    for (; u + 8 <= run; u += 8) {
+      float x[8];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) x[e] = (float)src[(u + e) * step];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) a += x[e];
     }
+    for (; u < run; ++u) a += (float)src[u * step];
     j += run;
     ++page;
     off = 0;
@@ -129,16 +135,27 @@ __global__ __launch_bounds__(256) void qk_norm_rows_kv_kernel(const T* __restric
   }
 }
 
+// Workgroup = (32 rows of the step, key / value head): every wave finds the rows that complete a block and
+// all threads average those blocks one after the other.
 template <typename T>
 __global__ __launch_bounds__(256) void pool_blocks_kernel(const T* __restrict__ k_cache, const T* __restrict__ v_cache,
-                                                          const int* __restrict__ slots, int G, int Dp, int Dvp, int bs,
-                                                          PoolArgs<T> pa) {
-  const long t = blockIdx.x;
-  const int s = pa.row_seq[t], p = pa.positions[t];
-  if (s < 0 || slots[t] < 0 || (p + 1) % pa.pool != 0) return;
-  const int* tab = pa.tables + (long)s * pa.max_blocks;
-  for (int i = threadIdx.x; i < G * (Dp + Dvp); i += 256)
-    pool_block(k_cache, v_cache, p, tab, i / (Dp + Dvp), G, Dp, Dvp, bs, pa, i % (Dp + Dvp));
+                                                          const int* __restrict__ slots, int T_, int G, int Dp, int Dvp,
+                                                          int bs, PoolArgs<T> pa) {
+  const int lane = threadIdx.x & 63, t = blockIdx.x * 32 + lane;
+  int s = -1, p = 0;
+  if (lane < 32 && t < T_) {
+    p = pa.positions[t];
+    s = slots[t] >= 0 && (p + 1) % pa.pool == 0 ? pa.row_seq[t] : -1;
+  }
+  unsigned long long todo = __ballot(s >= 0);
+  while (todo) {
+    const int l = __ffsll(todo) - 1;
+    todo &= todo - 1;
+    const int* tab = pa.tables + (long)__shfl(s, l) * pa.max_blocks;
+    const int pl = __shfl(p, l);
+    for (int i = threadIdx.x; i < Dp + Dvp; i += 256)
+      pool_block(k_cache, v_cache, pl, tab, (int)blockIdx.y, G, Dp, Dvp, bs, pa, i);
+  }
 }
 
 template <typename T>
@@ -179,12 +196,12 @@ void launch_pool_blocks(const void* k_cache, const void* v_cache, const int* tab
                         int T, int G, int Dp, int Dvp, int bs, bool f32, hipStream_t s) {
   if (T <= 0 || pool <= 0) return;
   if (f32)
-    pool_blocks_kernel<float><<<T, 256, 0, s>>>(
-        (const float*)k_cache, (const float*)v_cache, slots, G, Dp, Dvp, bs,
+    pool_blocks_kernel<float><<<dim3((T + 31) / 32, G), 256, 0, s>>>(
+        (const float*)k_cache, (const float*)v_cache, slots, T, G, Dp, Dvp, bs,
         {pool, pool_rows, max_blocks, (float*)k_pool, (float*)v_pool, positions, row_seq, tables});
   else
-    pool_blocks_kernel<bf16><<<T, 256, 0, s>>>(
-        (const bf16*)k_cache, (const bf16*)v_cache, slots, G, Dp, Dvp, bs,
+    pool_blocks_kernel<bf16><<<dim3((T + 31) / 32, G), 256, 0, s>>>(
+        (const bf16*)k_cache, (const bf16*)v_cache, slots, T, G, Dp, Dvp, bs,
         {pool, pool_rows, max_blocks, (bf16*)k_pool, (bf16*)v_pool, positions, row_seq, tables});
 }
 

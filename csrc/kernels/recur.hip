@@ -2,7 +2,9 @@
 // or f32; decays, step sizes, states and all recurrences are f32 in both):
 //   decay_chunk_kernel, decay_step_kernel   linear attention with a constant decay per head, S <- decay S +
 //                                           k v^T, o = S^T q, in chunks on the f32 matrix cores or row by row
-//   selective_scan_kernel                   S <- exp(dt A) S + dt x B, y = S C + d x, out = y silu(z)
+//   selective_scan_kernel, selective_step_kernel
+//                                           S <- exp(dt A) S + dt x B, y = S C + d x, out = y silu(z), over many
+//                                           rows per sequence or one row each (with dt's projection)
 //   row_norm_gate_kernel                    RMS norm of whole rows, times a sigmoid gate and a factor
 // Rows of a step are packed: sequence s owns rows row_cu[s] .. row_cu[s+1]; a sequence whose first row is at
 // position 0 starts from a zero state whatever its slot holds.
@@ -237,6 +239,7 @@ __global__ __launch_bounds__(256) void decay_step_kernel(const T* __restrict__ q
     const bool fresh = positions[t] == 0;
     f32x4 acc = {0.f, 0.f, 0.f, 0.f};
     if (c < Dv)
+#pragma unroll 8
       for (int d = dg; d < D; d += 16) {
         float* Sr = S + (long)d * Dv + c;
         f32x4 x = {0.f, 0.f, 0.f, 0.f};
@@ -277,12 +280,31 @@ __device__ __forceinline__ float quad_sum(float v) {
   return v;
 }
 
+// softplus, silu and exp(dt A) of the selective scan. FAST (bf16 activations): the hardware exp / log /
+// reciprocal, and for small e = exp(v) the series of log(1 + e), which keeps its relative accuracy there; a
+// true-f32 run uses the precise functions.
+template <bool FAST>
+__device__ __forceinline__ float softplus(float v) {
+  if (!FAST) return v > 20.f ? v : log1pf(expf(v));
+  const float e = __expf(v);
+  const float small = e * (1.f - e * (0.5f - e * (1.f / 3.f - e * 0.25f)));
+  return v > 20.f ? v : e < 0.03125f ? small : __logf(1.f + e);
+}
+template <bool FAST>
+__device__ __forceinline__ float silu_f(float v) {
+  if (FAST) return v * __builtin_amdgcn_rcpf(1.f + __expf(-v));
+  return v / (1.f + expf(-v));
+}
+constexpr float kLog2e = 1.4426950408889634f;
+
 // Selective scan. Workgroup = (sequence, 64 channels); the four lanes of a quad share a channel and keep NS
 // of its N states each in registers (N <= 4 NS; states past N have B = C = 0). Tokens are staged 16 at a
 // time: step sizes dt = softplus(dtr + bias), dt x, and the B and C rows go to LDS, the next block's inputs
 // travel to registers meanwhile; a token then costs NS exponentials and fused updates per lane and two
-// cross-lane moves, with no barrier inside the token loop. The outputs leave through LDS, where the skip
-// d x and the gate silu(z) are applied by the threads that hold x and z.
+// cross-lane moves, with no barrier inside the token loop. Rows past the sequence are staged with dt = 0
+// and x = 0 (they leave the state as it is), so the loop has a fixed length and its LDS reads are
+// scheduled ahead. The outputs leave through LDS, where the skip d x and the gate silu(z) are applied by
+// the threads that hold x and z.
 template <typename T, int NS>
 __global__ __launch_bounds__(256) void selective_scan_kernel(const T* __restrict__ x, long x_ld,
                                                              const float* __restrict__ dtr, long dt_ld,
@@ -313,14 +335,14 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(const T* __restrict
   }
   float* S = state + ((long)slot * C + ch) * N + qd * NS;
   const bool fresh = positions[r0] == 0;
-  constexpr float kLog2e = 1.4426950408889634f;
+  constexpr bool FAST = sizeof(T) == 2;
   float st[NS], A[NS];
 #pragma unroll
   for (int i = 0; i < NS; ++i) {
     const bool ok = ch < C && qd * NS + i < N;
     st[i] = (ok && !fresh) ? S[i] : 0.f;
     A[i] = ok ? -expf(a_log[(long)ch * N + qd * NS + i]) : 0.f;
-    if (sizeof(T) == 2) A[i] *= kLog2e;      // bf16 activations: hardware exp2 of (dt A log2 e)
+    if (FAST) A[i] *= kLog2e;      // exp2 of (dt A log2 e)
   }
   const float bias = cs < C ? dt_bias[cs] : 0.f, ds = cs < C ? dskip[cs] : 0.f;
   float rx[PT], rz[PT], rd[PT], rb[PB], rc[PB];
@@ -350,7 +372,7 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(const T* __restrict
 #pragma unroll
     for (int j = 0; j < PT; ++j) {
       const float av = rd[j] + bias;
-      const float dt = av > 20.f ? av : log1pf(expf(av));            // softplus
+      const float dt = tr + 4 * j >= nb ? 0.f : softplus<FAST>(av);
       sdt[tr + 4 * j][tid & 63] = dt;
       sdx[tr + 4 * j][tid & 63] = dt * rx[j];
       cx[j] = rx[j];
@@ -366,14 +388,15 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(const T* __restrict
     }
     __syncthreads();
     if (t0 + TB < r1) fetch(t0 + TB);        // in flight during the token loop
-    for (int tt = 0; tt < nb; ++tt) {
+#pragma unroll
+    for (int tt = 0; tt < TB; ++tt) {
       const float dt = sdt[tt][cl], dx = sdx[tt][cl];
       const float* pb = sB + tt * NP + qd * NS;
       const float* pc = sC + tt * NP + qd * NS;
       float y0 = 0.f, y1 = 0.f;
 #pragma unroll
       for (int i = 0; i < NS; ++i) {
-        const float a = sizeof(T) == 2 ? __builtin_amdgcn_exp2f(dt * A[i]) : expf(dt * A[i]);
+        const float a = FAST ? __builtin_amdgcn_exp2f(dt * A[i]) : expf(dt * A[i]);
         st[i] = fmaf(a, st[i], dx * pb[i]);
         if (i & 1) y1 = fmaf(st[i], pc[i], y1);
         else y0 = fmaf(st[i], pc[i], y0);
@@ -387,7 +410,7 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(const T* __restrict
       const int tt = tr + 4 * j;
       if (tt < nb && cs < C) {
         const float y = fmaf(ds, cx[j], sy[tt][tid & 63]);
-        out[(long)(t0 + tt) * C + cs] = (T)(y * (cz[j] / (1.f + expf(-cz[j]))));
+        out[(long)(t0 + tt) * C + cs] = (T)(y * silu_f<FAST>(cz[j]));
       }
     }
     // (the next block's staging overwrites sdt / sdx / sB / sC, which every wave finished reading at the
@@ -397,6 +420,93 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(const T* __restrict
 #pragma unroll
     for (int i = 0; i < NS; ++i)
       if (qd * NS + i < N) S[i] = st[i];
+  }
+}
+
+// Decoding: row s is sequence s's one row. Same workgroup shape and lanes as above; the step sizes' low-rank
+// projection dtr = W low (W [C, R], low [R] per row) happens here too, a quad sharing the dot product
+// of its channel.
+template <typename T, int NS>
+__global__ __launch_bounds__(256) void selective_step_kernel(const T* __restrict__ x, long x_ld,
+                                                             const T* __restrict__ low, long l_ld,
+                                                             const T* __restrict__ wdt, int R, int vec,
+                                                             const T* __restrict__ b, long b_ld,
+                                                             const T* __restrict__ cc, long c_ld,
+                                                             const T* __restrict__ z, long z_ld,
+                                                             const float* __restrict__ a_log,
+                                                             const float* __restrict__ dt_bias,
+                                                             const float* __restrict__ dskip,
+                                                             float* __restrict__ state,
+                                                             const int* __restrict__ state_slots,
+                                                             const int* __restrict__ positions, T* __restrict__ out,
+                                                             int C, int N) {
+  extern __shared__ __attribute__((aligned(16))) float slow[];      // [R]
+  constexpr bool FAST = sizeof(T) == 2;
+  const long t = blockIdx.x;
+  const int tid = threadIdx.x, cl = tid >> 2, qd = tid & 3, ch = blockIdx.y * 64 + cl;
+  const int slot = state_slots[t];
+  if (slot < 0) {      // padding row
+    if (ch < C && qd == 0) out[t * C + ch] = (T)0.f;
+    return;
+  }
+  const bool ok = ch < C, fresh = positions[t] == 0;
+  float* S = state + ((long)slot * C + ch) * N + qd * NS;
+  float st[NS], A[NS], bv[NS], cv[NS];
+#pragma unroll
+  for (int i = 0; i < NS; ++i) {
+    const bool in = ok && qd * NS + i < N;
+    st[i] = (in && !fresh) ? S[i] : 0.f;
+    A[i] = in ? a_log[(long)ch * N + qd * NS + i] : 0.f;
+    bv[i] = in ? (float)b[t * b_ld + qd * NS + i] : 0.f;
+    cv[i] = in ? (float)cc[t * c_ld + qd * NS + i] : 0.f;
+  }
+  const float xv = ok ? (float)x[t * x_ld + ch] : 0.f, zv = ok ? (float)z[t * z_ld + ch] : 0.f;
+  // (the first 128 columns of the projection's row travel to registers before the barrier)
+  typedef T t8 __attribute__((ext_vector_type(8)));
+  t8 w0[4];
+  const T* wr = wdt + (long)ch * R;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const int r = 8 * qd + 32 * j;
+    if (ok && vec && r < R) w0[j] = *reinterpret_cast<const t8*>(wr + r);
+    else w0[j] = t8((T)0.f);
+  }
+  for (int r = tid; r < R; r += 256) slow[r] = (float)low[t * l_ld + r];
+  __syncthreads();
+  float acc = 0.f;
+  if (ok) {
+    if (vec) {      // R % 8 == 0
+      float a1 = 0.f;
+      auto dot8 = [&](const t8& wv, int r) {
+        const f32x4 l0 = *reinterpret_cast<const f32x4*>(slow + r), l1 = *reinterpret_cast<const f32x4*>(slow + r + 4);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          acc = fmaf((float)wv[e], l0[e], acc);
+          a1 = fmaf((float)wv[4 + e], l1[e], a1);
+        }
+      };
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (8 * qd + 32 * j < R) dot8(w0[j], 8 * qd + 32 * j);
+      for (int r = 8 * qd + 128; r < R; r += 32) dot8(*reinterpret_cast<const t8*>(wr + r), r);
+      acc += a1;
+    } else {
+      for (int r = qd; r < R; r += 4) acc = fmaf((float)wr[r], slow[r], acc);
+    }
+  }
+  const float dt = ok ? softplus<FAST>(quad_sum(acc) + dt_bias[ch]) : 0.f, dx = dt * xv;
+  float y = 0.f;
+#pragma unroll
+  for (int i = 0; i < NS; ++i) {
+    const float a = FAST ? __builtin_amdgcn_exp2f(-dt * kLog2e * __expf(A[i])) : expf(-dt * expf(A[i]));
+    st[i] = fmaf(a, st[i], dx * bv[i]);
+    y = fmaf(st[i], cv[i], y);
+    if (ok && qd * NS + i < N) S[i] = st[i];
+  }
+  y = quad_sum(y);
+  if (ok && qd == 0) {
+    y = fmaf(dskip[ch], xv, y);
+    out[t * C + ch] = (T)(y * silu_f<FAST>(zv));
   }
 }
 
@@ -479,6 +589,28 @@ void decay_scan_t(const T* q, long q_ld, const T* k, long k_ld, const T* v, long
 }
 
 template <typename T>
+int selective_step_t(const T* x, long x_ld, const T* low, long l_ld, const T* wdt, int R, const T* b, long b_ld, const T* c,
+                     long c_ld, const T* z, long z_ld, const float* a_log, const float* dt_bias, const float* d, float* state,
+                     const int* state_slots, const int* positions, T* out, int T_, int C, int N, hipStream_t s) {
+  dim3 grid(T_, (C + 63) / 64);
+  const int vec = R % 8 == 0 && reinterpret_cast<uintptr_t>(wdt) % (8 * sizeof(T)) == 0;
+#define BFLY_SST(NS)                                                                                                  \
+  selective_step_kernel<T, NS><<<grid, 256, R * sizeof(float), s>>>(x, x_ld, low, l_ld, wdt, R, vec, b, b_ld, c, c_ld, z, \
+                                                                    z_ld, a_log, dt_bias, d, state, state_slots, positions, \
+                                                                    out, C, N)
+  if (N <= 4) BFLY_SST(1);
+  else if (N <= 8) BFLY_SST(2);
+  else if (N <= 16) BFLY_SST(4);
+  else if (N <= 32) BFLY_SST(8);
+  else if (N <= 64) BFLY_SST(16);
+  else if (N <= 128) BFLY_SST(32);
+  else if (N <= 256) BFLY_SST(64);
+  else return -1;
+#undef BFLY_SST
+  return 0;
+}
+
+template <typename T>
 int selective_scan_t(const T* x, long x_ld, const float* dtr, long dt_ld, const T* b, long b_ld, const T* c, long c_ld,
                      const T* z, long z_ld, const float* a_log, const float* dt_bias, const float* d, float* state,
                      const int* state_slots, const int* row_cu, int nseq, const int* positions, T* out, int C, int N,
@@ -537,6 +669,20 @@ int launch_selective_scan(const void* x, long x_ld, const float* dtr, long dt_ld
                                    (float*)out, C, N, s);
   return selective_scan_t<bf16>((const bf16*)x, x_ld, dtr, dt_ld, (const bf16*)b, b_ld, (const bf16*)c, c_ld, (const bf16*)z,
                                 z_ld, a_log, dt_bias, d, state, state_slots, row_cu, nseq, positions, (bf16*)out, C, N, s);
+}
+
+int launch_selective_step(const void* x, long x_ld, const void* low, long l_ld, const void* wdt, int R, const void* b,
+                          long b_ld, const void* c, long c_ld, const void* z, long z_ld, const float* a_log,
+                          const float* dt_bias, const float* d, float* state, const int* state_slots, const int* positions,
+                          void* out, int T, int C, int N, bool f32, hipStream_t s) {
+  if (T <= 0) return 0;
+  if (f32)
+    return selective_step_t<float>((const float*)x, x_ld, (const float*)low, l_ld, (const float*)wdt, R, (const float*)b, b_ld,
+                                   (const float*)c, c_ld, (const float*)z, z_ld, a_log, dt_bias, d, state, state_slots,
+                                   positions, (float*)out, T, C, N, s);
+  return selective_step_t<bf16>((const bf16*)x, x_ld, (const bf16*)low, l_ld, (const bf16*)wdt, R, (const bf16*)b, b_ld,
+                                (const bf16*)c, c_ld, (const bf16*)z, z_ld, a_log, dt_bias, d, state, state_slots, positions,
+                                (bf16*)out, T, C, N, s);
 }
 
 }  // namespace bfly
