@@ -412,18 +412,25 @@ def sample(logits, temps=None, seeds=None, vstart: int = 0, out_ids=None, out_sc
     if out_scores is None:
         out_scores = _empty(rows, dtype=torch.float32, device=logits.device)
     if logits.dtype == torch.float32:
-        # f32 serving mode: greedy rows pick from the f32 values themselves; stochastic rows go
-        # through the bf16 sampler on a rounded copy (16-byte rows)
-        if temps is None and thresh is None:
+        # f32 logits: the choice is made from the f32 values themselves; rows restricted by top-k / top-p
+        # (whose thresholds are values of a rounded copy) go through that copy
+        odd = logits.stride(0) % 4 != 0 or logits.data_ptr() % 16 != 0
+        if temps is None and thresh is None and odd:
             torch.ops.bfly.sample_greedy_f32(logits, vstart, out_ids, out_scores, check_finite)
             return out_ids, out_scores
-        n = logits.shape[1]
-        buf = torch.empty(rows, (n + 7) // 8 * 8, dtype=torch.bfloat16, device=logits.device)
-        buf[:, :n].copy_(logits)
-        logits = buf[:, :n]
+        if thresh is not None or odd:
+            logits = _bf16_rows(logits)
     ws = _arena.get(logits.device, "sample", rows * 64, torch.int64)
     torch.ops.bfly.sample(logits, temps, seeds, vstart, out_ids, out_scores, ws, thresh, check_finite)
     return out_ids, out_scores
+
+
+def _bf16_rows(logits):
+    """A bf16 copy of f32 logits in 16-byte rows."""
+    rows, n = logits.shape
+    buf = torch.empty(rows, (n + 7) // 8 * 8, dtype=torch.bfloat16, device=logits.device)
+    buf[:, :n].copy_(logits)
+    return buf[:, :n]
 
 
 def topkp_threshold(logits, temps, top_k, top_p, reduce_sum=None, reduce_max=None,
@@ -435,6 +442,8 @@ def topkp_threshold(logits, temps, top_k, top_p, reduce_sum=None, reduce_max=Non
     thresh [R] f32 (-inf = unfiltered row), the `thresh` argument of `sample`."""
     if not _gpu(logits):
         return ref.topkp_threshold(logits, temps, top_k, top_p, reduce_sum, reduce_max, use_k, use_p)
+    if logits.dtype == torch.float32:
+        logits = _bf16_rows(logits)
     R = logits.shape[0]
     L = torch.ops.bfly
     ws = _arena.get(logits.device, "tkp", R * 521, torch.float32)[: R * 521]

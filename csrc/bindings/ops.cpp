@@ -248,8 +248,10 @@ void sample(const Tensor& logits, const c10::optional<Tensor>& temps,
             const c10::optional<Tensor>& seeds, int64_t vstart, Tensor& out_ids,
             Tensor& out_scores, Tensor& workspace, const c10::optional<Tensor>& thresh,
             bool check_finite) {
-  CHECK_GPU(logits); CHECK_BF16(logits);
-  TORCH_CHECK(logits.dim() == 2 && logits.stride(1) == 1 && logits.stride(0) % 8 == 0, "sample: logits");
+  CHECK_GPU(logits);
+  const bool f32 = logits.scalar_type() == at::kFloat;
+  TORCH_CHECK(f32 || logits.scalar_type() == at::kBFloat16, "sample: bf16 or f32 logits");
+  TORCH_CHECK(logits.dim() == 2 && logits.stride(1) == 1 && logits.stride(0) % (f32 ? 4 : 8) == 0, "sample: logits");
   CHECK_ALIGN16(logits);
   const int rows = logits.size(0), V = logits.size(1);
   CHECK_I32(out_ids);
@@ -274,7 +276,7 @@ void sample(const Tensor& logits, const c10::optional<Tensor>& temps,
     thp = thresh->data_ptr<float>();
   }
   c10::DeviceGuard g(logits.device());
-  bfly::launch_sample(bf(logits), logits.stride(0), rows, V, vstart, tp, sp,
+  bfly::launch_sample(logits.data_ptr(), f32, logits.stride(0), rows, V, vstart, tp, sp,
                       reinterpret_cast<uint64_t*>(workspace.data_ptr()), out_ids.data_ptr<int>(),
                       out_scores.data_ptr<float>(), cur_stream(), thp, check_finite ? 1 : 0);
 }

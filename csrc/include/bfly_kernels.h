@@ -94,7 +94,7 @@ void launch_gather_rows(const void* src, long src_ld, const void* idx, bool idx6
 
 // sample.hip
 constexpr int kSampleMaxChunks = 64;
-void launch_sample(const bf16* logits, long row_stride, int rows, int V, int vstart,
+void launch_sample(const void* logits, bool f32, long row_stride, int rows, int V, int vstart,
                    const float* temps, const long* seeds, uint64_t* workspace, int* out_ids,
                    float* out_scores, hipStream_t stream, const float* thresh = nullptr,
                    int check_finite = 0);

@@ -53,8 +53,32 @@ __device__ __forceinline__ uint64_t wave_max_u64(uint64_t v) {
   return v;
 }
 
+// Eight logits from i on as f32, and whether one of them is Inf or NaN (exponent all ones).
+__device__ __forceinline__ void load8_logits(const bf16* p, float (&s)[8], uint32_t& nonfinite) {
+  const u32x4 raw = *reinterpret_cast<const u32x4*>(p);
+#pragma unroll
+  for (int k = 0; k < 4; ++k)
+    nonfinite |= (uint32_t)((raw[k] & 0x7F80u) == 0x7F80u) | (uint32_t)((raw[k] & 0x7F800000u) == 0x7F800000u);
+  const bf16x8 v = __builtin_bit_cast(bf16x8, raw);
+#pragma unroll
+  for (int j = 0; j < 8; ++j) s[j] = bf2f(v[j]);
+}
+__device__ __forceinline__ void load8_logits(const float* p, float (&s)[8], uint32_t& nonfinite) {
+#pragma unroll
+  for (int k = 0; k < 2; ++k) {
+    const f32x4 v = *reinterpret_cast<const f32x4*>(p + 4 * k);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      nonfinite |= (uint32_t)((__float_as_uint(v[j]) & 0x7F800000u) == 0x7F800000u);
+      s[4 * k + j] = v[j];
+    }
+  }
+}
+
+// T: bf16, or float for models whose logits are f32 (the same choice from the unrounded values).
+template <typename T>
 __global__ void __launch_bounds__(kSampleThreads)
-sample_partial_kernel(const bf16* __restrict__ logits, long row_stride, int V, int chunk,
+sample_partial_kernel(const T* __restrict__ logits, long row_stride, int V, int chunk,
                       int vstart, const float* __restrict__ temps,
                       const long* __restrict__ seeds, const float* __restrict__ thresh,
                       uint64_t* __restrict__ partial, int check_finite) {
@@ -68,19 +92,16 @@ sample_partial_kernel(const bf16* __restrict__ logits, long row_stride, int V, i
   const uint64_t seed = seeds ? (uint64_t)seeds[row] : 0;
   const float thr = (thresh != nullptr && !greedy) ? thresh[row] : -INFINITY;
   const int begin = c * chunk, end = min(V, begin + chunk);
-  const bf16* lr = logits + (long)row * row_stride;
+  const T* lr = logits + (long)row * row_stride;
   uint64_t best = 0;
-  uint32_t nonfinite = 0;   // OR of exponent-all-ones tests (Inf / NaN bf16)
+  uint32_t nonfinite = 0;   // OR of exponent-all-ones tests (Inf / NaN)
   for (int i = begin + threadIdx.x * 8; i < end; i += kSampleThreads * 8) {
     if (i + 8 <= end) {
-      const u32x4 raw = *reinterpret_cast<const u32x4*>(lr + i);
-#pragma unroll
-      for (int k = 0; k < 4; ++k)   // bf16 exponent all ones: Inf or NaN
-        nonfinite |= (uint32_t)((raw[k] & 0x7F80u) == 0x7F80u) | (uint32_t)((raw[k] & 0x7F800000u) == 0x7F800000u);
-      const bf16x8 v = __builtin_bit_cast(bf16x8, raw);
+      float v[8];
+      load8_logits(lr + i, v, nonfinite);
 #pragma unroll
       for (int j = 0; j < 8; ++j) {
-        float s = bf2f(v[j]);
+        float s = v[j];
         if (!greedy) {
           s = s * inv_t;
           if (s < thr) continue;            // outside the top-k / top-p set
@@ -91,9 +112,8 @@ sample_partial_kernel(const bf16* __restrict__ logits, long row_stride, int V, i
       }
     } else {
       for (int j = 0; i + j < end; ++j) {
-        const uint32_t bits = reinterpret_cast<const uint16_t*>(lr)[i + j];
-        nonfinite |= (uint32_t)((bits & 0x7F80u) == 0x7F80u);
-        float s = bf2f(lr[i + j]);
+        float s = (float)lr[i + j];
+        nonfinite |= (uint32_t)((__float_as_uint(s) & 0x7F800000u) == 0x7F800000u);
         if (!greedy) {
           s = s * inv_t;
           if (s < thr) continue;
@@ -469,7 +489,7 @@ void launch_sample_greedy_f32(const float* logits, long row_stride, int rows, in
   sample_greedy_f32_kernel<<<rows, 1024, 0, stream>>>(logits, row_stride, V, vstart, out_ids, out_scores, check_finite);
 }
 
-void launch_sample(const bf16* logits, long row_stride, int rows, int V, int vstart,
+void launch_sample(const void* logits, bool f32, long row_stride, int rows, int V, int vstart,
                    const float* temps, const long* seeds, uint64_t* workspace, int* out_ids,
                    float* out_scores, hipStream_t stream, const float* thresh, int check_finite) {
   if (rows <= 0) return;
@@ -479,8 +499,12 @@ void launch_sample(const bf16* logits, long row_stride, int rows, int V, int vst
   chunk = (chunk + 7) / 8 * 8;
   chunks = (V + chunk - 1) / chunk;
   dim3 g1(rows, chunks);
-  sample_partial_kernel<<<g1, kSampleThreads, 0, stream>>>(logits, row_stride, V, chunk, vstart,
-                                                           temps, seeds, thresh, workspace, check_finite);
+  if (f32)
+    sample_partial_kernel<float><<<g1, kSampleThreads, 0, stream>>>((const float*)logits, row_stride, V, chunk, vstart,
+                                                                    temps, seeds, thresh, workspace, check_finite);
+  else
+    sample_partial_kernel<bf16><<<g1, kSampleThreads, 0, stream>>>((const bf16*)logits, row_stride, V, chunk, vstart,
+                                                                   temps, seeds, thresh, workspace, check_finite);
   sample_final_kernel<<<rows, 64, 0, stream>>>(workspace, chunks, vstart, out_ids, out_scores);
 }
 

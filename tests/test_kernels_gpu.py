@@ -117,6 +117,44 @@ def test_sample_gumbel_matches_reference():
     assert ids.cpu().tolist() == ids_ref.tolist()
 
 
+@pytest.mark.parametrize("V,pad", [(1000, 0), (4096, 128), (61, 67), (61, 2), (32000, 0)])
+def test_sample_f32_logits(V, pad):
+    """f32 logits (also a view of padded rows): greedy rows, with and without a temperature vector beside
+    them, pick from the unrounded values (two that one bf16 value would merge, the higher index larger),
+    stochastic rows match the reference on the f32 values, Inf / NaN rows are marked."""
+    g = torch.Generator().manual_seed(V + pad)
+    wide = torch.randn(5, V + pad, generator=g).to(DEV)
+    wide[:, V:] = 50.0                                   # padding must never win
+    lg = wide[:, :V]
+    lg[:, 7], lg[:, V - 3] = 16.3342, 16.3889
+    temps = torch.tensor([0.0, 0.7, 0.0, 30.0, 0.0], device=DEV)
+    seeds = torch.tensor([1, 42, 5, 12345, 9], dtype=torch.int64, device=DEV)
+    assert ops.sample(lg)[0].tolist() == [V - 3] * 5
+    ids, sc = ops.sample(lg, temps, seeds)
+    aligned = (V + pad) % 4 == 0
+    if aligned:
+        assert [int(ids[r]) for r in (0, 2, 4)] == [V - 3] * 3 and abs(float(sc[0]) - 16.3889) < 1e-5
+        assert ids.tolist() == ref.sample(lg.cpu(), temps.cpu(), seeds.cpu(), vstart=0)[0].tolist()
+    lg[2, V // 2] = float("nan")
+    lg[4, 3] = float("inf")
+    ids = ops.sample(lg, temps, seeds, check_finite=True)[0].tolist()
+    assert ids[2] == ids[4] == -1 and min(ids[0], ids[1], ids[3]) >= 0
+
+
+def test_sample_topk_topp_takes_f32_logits():
+    from butterfly_amd.engine.sampler import Sampler, SamplingParams
+
+    V = 500
+    lg = torch.zeros(3, 512, device=DEV)
+    lg[:, :V] = torch.randn(3, V, generator=torch.Generator().manual_seed(3)).to(DEV)
+    params = [SamplingParams(temperature=0.8, top_k=3), SamplingParams(temperature=1.0, top_p=0.05), SamplingParams(temperature=0.0)]
+    temps = torch.tensor([p.temperature for p in params], device=DEV)
+    seeds = torch.arange(3, dtype=torch.int64, device=DEV)
+    ids = Sampler(None, V, 0, 1).sample(lg, temps, seeds, params).tolist()
+    rank = [int((lg[r, :V] > lg[r, ids[r]]).sum()) for r in range(3)]
+    assert rank[0] <= 3 and rank[1] <= 10 and rank[2] == 0
+
+
 def test_sample_topk_topp_on_device():
     """Filtered sampling on the GPU: the radix-select thresholds (tkp_* kernels) equal the
     tie-aware exact ones on a 128k vocabulary with high-entropy rows (nuclei of thousands of
