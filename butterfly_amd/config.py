@@ -434,7 +434,7 @@ def _attention_sizes(index: int, m: dict) -> dict:
     H, D = int(m["heads"]), int(m["dim"])
     mask = m.get("mask") or {}
     sp = {"heads": H, "kv_heads": int(m.get("kv_heads", H)), "dim": D, "vdim": int(m.get("vdim", D)),
-          "scale": float(m.get("scale", D ** -0.5)), "window": int(mask.get("size", 1 << 30)),
+          "scale": float(m.get("scale", D ** -0.5)), "window": int(mask.get("size") or 1 << 30),
           "pool": int(mask.get("pool") or 0)}
     if sp["kv_heads"] < 1 or H % sp["kv_heads"] or min(D, sp["vdim"], sp["window"]) < 1 or sp["pool"] < 0:
         raise ValueError(f"layer {index}: bad attention sizes")

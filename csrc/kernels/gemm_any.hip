@@ -270,7 +270,8 @@ __global__ __launch_bounds__(256) void moe_sum4_kernel(const float* __restrict__
 
 // Router logits of a small step (a few rows): one wave per (token, expert), lanes split the
 // hidden dim, f32 accumulation. Large steps use the f32-output GEMM instead.
-template <typename T>
+// V = 8: eight elements per access (Hd and ldx multiples of 8, aligned rows).
+template <typename T, int V>
 __global__ __launch_bounds__(256) void router_logits_kernel(const T* __restrict__ x, long ldx,
                                                             const T* __restrict__ wr, float* __restrict__ logits,
                                                             int E, int Hd) {
@@ -279,7 +280,22 @@ __global__ __launch_bounds__(256) void router_logits_kernel(const T* __restrict_
   const T* xr = x + (long)t * ldx;
   const T* w = wr + (long)e * Hd;
   float a = 0.f;
-  for (int k = lane; k < Hd; k += 64) a = fmaf(ldf(xr + k), ldf(w + k), a);
+  if (V > 1) {
+    typedef T tv __attribute__((ext_vector_type(V)));
+    float b = 0.f;
+#pragma unroll 4
+    for (int k = V * lane; k < Hd; k += V * 64) {
+      const tv xv = *reinterpret_cast<const tv*>(xr + k), wv = *reinterpret_cast<const tv*>(w + k);
+#pragma unroll
+      for (int e = 0; e < V; e += 2) {
+        a = fmaf((float)xv[e], (float)wv[e], a);
+        b = fmaf((float)xv[e + 1], (float)wv[e + 1], b);
+      }
+    }
+    a += b;
+  } else {
+    for (int k = lane; k < Hd; k += 64) a = fmaf(ldf(xr + k), ldf(w + k), a);
+  }
   a = wave_sum(a);
   if (lane == 0) logits[(long)t * E + e] = a;
 }
@@ -681,8 +697,13 @@ void launch_router_logits(const void* x, long ldx, const void* wr, float* logits
                           hipStream_t s) {
   if (T <= 0) return;
   dim3 grid(T, (E + 3) / 4);
-  if (f32) router_logits_kernel<float><<<grid, 256, 0, s>>>((const float*)x, ldx, (const float*)wr, logits, E, Hd);
-  else router_logits_kernel<bf16><<<grid, 256, 0, s>>>((const bf16*)x, ldx, (const bf16*)wr, logits, E, Hd);
+  const size_t al = f32 ? 32 : 16;
+  const bool vec = Hd % 8 == 0 && ldx % 8 == 0 && reinterpret_cast<uintptr_t>(x) % al == 0 &&
+                   reinterpret_cast<uintptr_t>(wr) % al == 0;
+#define BFLY_RL(TT, V) router_logits_kernel<TT, V><<<grid, 256, 0, s>>>((const TT*)x, ldx, (const TT*)wr, logits, E, Hd)
+  if (f32) { if (vec) BFLY_RL(float, 8); else BFLY_RL(float, 1); }
+  else { if (vec) BFLY_RL(bf16, 8); else BFLY_RL(bf16, 1); }
+#undef BFLY_RL
 }
 
 void launch_moe_topk_scores(const float* logits, const float* bias, int top_k, int scoring, bool renorm, int* ids,

@@ -774,6 +774,18 @@ def test_requests_share_the_pages_of_a_common_prefix(target, tmp_path):
                   lambda t: ref.replay_step([(1000, t, list(range(len(t))))], [1000]).cpu().double())
 
 
+def test_a_stack_of_recurrent_layers_only(target, tmp_path):
+    """No attention layer: no pages to fill, only state slots."""
+    dev, dt = target
+    cfg = O.config([O.mamba_layer(24, 4, 3, 4, O.dense(16)), O.mamba_layer(8, 2, 2, 2, None)], 16, 40, 1e-5)
+    W = O.random_weights(cfg, seed=15)
+    toks = tokens_of(cfg, 60, 3)
+    eng = make_engine(tmp_path, cfg, W, dev, dt, cache_tokens=64)
+    assert eng.kv.layers == []
+    got = replay(eng, {"r": toks}, [[("r", 20)]] + [[("r", 1)]] * 8 + [[("r", 30)], [("r", 2)]])["r"]
+    assert_rows(got, O.forward(cfg, W, toks), dt)
+
+
 def test_page_copies_take_the_block_means_along():
     """A forked page (copy on write) carries every per-page tensor of its layer."""
     from butterfly_amd.engine.kv_cache import KVCache
@@ -808,7 +820,7 @@ def test_random_init_and_registry():
     assert [len(o) for o in out] == [3, 3]
     n = sum(math.prod(lp.global_shape) for lp in m.logical_params())
     assert abs(mc.param_count() - n) <= 5 * 24 + len(mc.layer_specs)          # (layer average rounded down, norms)
-    for change in ({"mask": {"size": 0}}, {"kv_heads": 2}):
+    for change in ({"mask": {"size": -1}}, {"kv_heads": 2}):
         bad = cfg_b()
         bad["layers"][3]["mixer"].update(change)
         with pytest.raises(ValueError):
