@@ -17,7 +17,13 @@ namespace bfly {
 
 namespace {
 
-__device__ __forceinline__ float act_in(float v, int act) { return act == 1 ? v / (1.f + expf(-v)) : v; }
+// an input's activation; FAST (bf16 inputs): hardware exp and reciprocal
+template <bool FAST>
+__device__ __forceinline__ float act_in(float v, int act) {
+  if (act != 1) return v;
+  if (FAST) return v * __builtin_amdgcn_rcpf(1.f + __expf(-v));
+  return v / (1.f + expf(-v));
+}
 
 // element 4 j .. 4 j + 3 of a row, zeros from n on
 template <typename T>
@@ -89,33 +95,55 @@ __global__ __launch_bounds__(256) void decay_chunk_kernel(const T* __restrict__ 
       st[i][e] = (!fresh && live && d < D) ? S[(long)d * Dv] : 0.f;
     }
   for (int i = tid; i <= C; i += 256) sd[i] = dpow[(long)h * n_pow + i];
+  // A chunk's inputs travel to registers as they are stored while the chunk before is computed (rows past the
+  // sequence: its last row again, so no load hangs on a branch; staged as zeros).
+  typedef T t4 __attribute__((ext_vector_type(4)));
+  constexpr int NQ = (C * (DP / 4) + 255) / 256, NV = C * 16 / 256;
+  t4 rq[NQ], rk[NQ], rv[NV];
+  auto fetch4 = [&](const T* row, int c, int size, bool v4) {
+    if (v4) return *reinterpret_cast<const t4*>(row + min(c, size - 4));
+    t4 r;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) r[e] = row[min(c + e, size - 1)];
+    return r;
+  };
+  auto fetch = [&](int t0) {
+#pragma unroll
+    for (int j = 0; j < NQ; ++j) {
+      const int i = tid + 256 * j, d = 4 * (i % (DP / 4));
+      const long t = min(t0 + i / (DP / 4), r1 - 1);
+      rq[j] = fetch4(q + t * q_ld + (long)h * D, d, D, vec & 1);
+      rk[j] = fetch4(k + t * k_ld + (long)h * D, d, D, vec & 1);
+    }
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+      const int i = tid + 256 * j;
+      const long t = min(t0 + (i >> 4), r1 - 1);
+      rv[j] = fetch4(v + t * v_ld + (long)h * Dv, c0 + 4 * (i & 15), Dv, vec & 2);
+    }
+  };
+  auto stage4 = [&](const t4& r, bool row, int c, int size) {
+    f32x4 a;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) a[e] = (row && c + e < size) ? act_in<sizeof(T) == 2>((float)r[e], act) : 0.f;
+    return a;
+  };
+  fetch(r0);
   for (int t0 = r0; t0 < r1; t0 += C) {
     const int n = min(C, r1 - t0);
-    for (int i = tid; i < C * (DP / 4); i += 256) {
-      const int t = i / (DP / 4), d = 4 * (i % (DP / 4));
-      f32x4 a = {0.f, 0.f, 0.f, 0.f}, b = {0.f, 0.f, 0.f, 0.f};
-      if (t < n) {
-        a = load4(q + (long)(t0 + t) * q_ld + (long)h * D, d, D, vec & 1);
-        b = load4(k + (long)(t0 + t) * k_ld + (long)h * D, d, D, vec & 1);
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          a[e] = act_in(a[e], act);
-          b[e] = act_in(b[e], act);
-        }
-      }
-      *reinterpret_cast<f32x4*>(sq + t * KP + d) = a;
-      *reinterpret_cast<f32x4*>(sk + t * KP + d) = b;
+    for (int j = 0; j < NQ; ++j) {
+      const int i = tid + 256 * j, t = i / (DP / 4), d = 4 * (i % (DP / 4));
+      if (NQ * 256 != C * (DP / 4) && t >= C) break;
+      *reinterpret_cast<f32x4*>(sq + t * KP + d) = stage4(rq[j], t < n, d, D);
+      *reinterpret_cast<f32x4*>(sk + t * KP + d) = stage4(rk[j], t < n, d, D);
     }
-    for (int i = tid; i < C * 16; i += 256) {
-      const int t = i >> 4, c = 4 * (i & 15);
-      f32x4 a = {0.f, 0.f, 0.f, 0.f};
-      if (t < n) {
-        a = load4(v + (long)(t0 + t) * v_ld + (long)h * Dv, c0 + c, Dv, vec & 2);
 #pragma unroll
-        for (int e = 0; e < 4; ++e) a[e] = act_in(a[e], act);
-      }
-      *reinterpret_cast<f32x4*>(sv + t * VP + c) = a;
+    for (int j = 0; j < NV; ++j) {
+      const int i = tid + 256 * j, t = i >> 4, c = 4 * (i & 15);
+      *reinterpret_cast<f32x4*>(sv + t * VP + c) = stage4(rv[j], t < n, c0 + c, Dv);
     }
+    if (t0 + C < r1) fetch(t0 + C);      // in flight during the products below
     __syncthreads();
     // (q . k) decay^(t - j): the tiles at or below the diagonal, dealt to the waves
     for (int tile = wave; tile < TT * (TT + 1) / 2; tile += 4) {
@@ -229,12 +257,12 @@ __global__ __launch_bounds__(256) void decay_step_kernel(const T* __restrict__ q
   const bool sv4 = (vec & 4) && c + 3 < Dv;      // 16-byte state rows
   for (int t = r0; t < r1; ++t) {
     for (int d = tid; d < D; d += 256) {
-      sq[d] = act_in((float)q[(long)t * q_ld + (long)h * D + d], act);
-      sk[d] = act_in((float)k[(long)t * k_ld + (long)h * D + d], act);
+      sq[d] = act_in<sizeof(T) == 2>((float)q[(long)t * q_ld + (long)h * D + d], act);
+      sk[d] = act_in<sizeof(T) == 2>((float)k[(long)t * k_ld + (long)h * D + d], act);
     }
     f32x4 vv = load4(v + (long)t * v_ld + (long)h * Dv, c, Dv, vec & 2);
 #pragma unroll
-    for (int e = 0; e < 4; ++e) vv[e] = act_in(vv[e], act);
+    for (int e = 0; e < 4; ++e) vv[e] = act_in<sizeof(T) == 2>(vv[e], act);
     __syncthreads();
     const bool fresh = positions[t] == 0;
     f32x4 acc = {0.f, 0.f, 0.f, 0.f};
@@ -345,24 +373,25 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(const T* __restrict
     if (FAST) A[i] *= kLog2e;      // exp2 of (dt A log2 e)
   }
   const float bias = cs < C ? dt_bias[cs] : 0.f, ds = cs < C ? dskip[cs] : 0.f;
-  float rx[PT], rz[PT], rd[PT], rb[PB], rc[PB];
+  // the next block's inputs as they are stored (rows and columns past the end: the last one again, so no
+  // load hangs on a branch; such values meet dt = 0 or B = C = 0)
+  T rx[PT], rz[PT], rb[PB], rc[PB];
+  float rd[PT];
+  const int csc = min(cs, C - 1);
   auto fetch = [&](int t0) {
-    const int nb = min(TB, r1 - t0);
 #pragma unroll
     for (int j = 0; j < PT; ++j) {
-      const int tt = tr + 4 * j;
-      const long t = t0 + tt;
-      const bool ok = tt < nb && cs < C;
-      rx[j] = ok ? (float)x[t * x_ld + cs] : 0.f;
-      rz[j] = ok ? (float)z[t * z_ld + cs] : 0.f;
-      rd[j] = ok ? dtr[t * dt_ld + cs] : 0.f;
+      const long t = min(t0 + tr + 4 * j, r1 - 1);
+      rx[j] = x[t * x_ld + csc];
+      rz[j] = z[t * z_ld + csc];
+      rd[j] = dtr[t * dt_ld + csc];
     }
 #pragma unroll
     for (int j = 0; j < PB; ++j) {
-      const int i = tid + 256 * j, tt = i / NP, n = i - tt * NP;
-      const bool ok = tt < nb && n < N;
-      rb[j] = ok ? (float)b[(long)(t0 + tt) * b_ld + n] : 0.f;
-      rc[j] = ok ? (float)cc[(long)(t0 + tt) * c_ld + n] : 0.f;
+      const int i = tid + 256 * j, tt = i / NP, n = min(i - tt * NP, N - 1);
+      const long t = min(t0 + tt, r1 - 1);
+      rb[j] = b[t * b_ld + n];
+      rc[j] = cc[t * c_ld + n];
     }
   };
   fetch(r0);
@@ -371,23 +400,24 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(const T* __restrict
     float cx[PT], cz[PT];
 #pragma unroll
     for (int j = 0; j < PT; ++j) {
-      const float av = rd[j] + bias;
-      const float dt = tr + 4 * j >= nb ? 0.f : softplus<FAST>(av);
+      const float dt = tr + 4 * j < nb ? softplus<FAST>(rd[j] + bias) : 0.f;
+      cx[j] = (float)rx[j];
+      cz[j] = (float)rz[j];
       sdt[tr + 4 * j][tid & 63] = dt;
-      sdx[tr + 4 * j][tid & 63] = dt * rx[j];
-      cx[j] = rx[j];
-      cz[j] = rz[j];
+      sdx[tr + 4 * j][tid & 63] = dt * cx[j];
     }
 #pragma unroll
     for (int j = 0; j < PB; ++j) {
       const int i = tid + 256 * j;
       if (i < TB * NP) {
-        sB[i] = rb[j];
-        sC[i] = rc[j];
+        const bool in = i % NP < N;
+        sB[i] = in ? (float)rb[j] : 0.f;
+        sC[i] = in ? (float)rc[j] : 0.f;
       }
     }
     __syncthreads();
     if (t0 + TB < r1) fetch(t0 + TB);        // in flight during the token loop
+    float ys[TB / 4];      // lane qd of a quad keeps the outputs of tokens qd, qd + 4, ... (no store in the loop)
 #pragma unroll
     for (int tt = 0; tt < TB; ++tt) {
       const float dt = sdt[tt][cl], dx = sdx[tt][cl];
@@ -402,8 +432,11 @@ __global__ __launch_bounds__(256) void selective_scan_kernel(const T* __restrict
         else y0 = fmaf(st[i], pc[i], y0);
       }
       const float y = quad_sum(y0 + y1);
-      if (qd == 0) sy[tt][cl] = y;
+      if ((tt & 3) == 0) ys[tt >> 2] = y;
+      else ys[tt >> 2] = qd == (tt & 3) ? y : ys[tt >> 2];
     }
+#pragma unroll
+    for (int j = 0; j < TB / 4; ++j) sy[4 * j + qd][cl] = ys[j];
     __syncthreads();
 #pragma unroll
     for (int j = 0; j < PT; ++j) {
