@@ -17,6 +17,7 @@ from typing import Any, Optional
 class ModelConfig:
     name: str
     arch: str                       # "llama" | "gpt2" | "mixtral" | "nesizen" | "zinesun" | "lizizen" | "gevipel" | "vuladra"
+                                # | "rumedra"
     vocab_size: int
     hidden_size: int
     intermediate_size: int
@@ -105,7 +106,7 @@ class ModelConfig:
                     if sp["type"] == "latent_attention") + \
                 sum(sp["kv_heads"] * (sp["maps"] * sp["dim"] + sp["vdim"]) * dtype_bytes for sp in runs
                     if sp["type"] in ("biased_attention", "diff_attention", "sloped_attention", "pooled_attention",
-                                      "side_by_side"))
+                                      "side_by_side", "attention_retention"))
         return 2 * self.num_layers * self.kv_size * dtype_bytes
 
     # ---- (de)serialisation -------------------------------------------------------------
@@ -273,6 +274,32 @@ class ModelConfig:
                    experts_per_token=max([f["top"] for f in moe] + [0]), layer_specs=specs)
 
     @classmethod
+    def from_rumedra(cls, js: dict, name: str = "rumedra") -> "ModelConfig":
+        """Map a Rumedra config.json ("architecture": "Rumedra") to ModelConfig: pre-norm layers over two
+        mixers (rotated windowed attention beside retention, "parallel"; linear attention whose forget gate
+        also decides what is written, "hgrn2"), dense ReLU GLUs or routed silu GLUs chosen inside the best
+        groups of experts, with identity experts and a shared one, a scaled embedding whose table is also the
+        LM head. Every size and per-layer constant is taken from the file."""
+        kinds = {"parallel": "attention_retention", "hgrn2": "hgrn"}
+        specs = []
+        for i, L in enumerate(js["layers"]):
+            if L["type"] not in kinds:
+                raise ValueError(f"layer {i}: Rumedra has no mixer {L['type']!r}")
+            specs.append(layer_spec(i, {**L, "type": kinds[L["type"]]}))
+        mx = lambda key: max([sp.get(key) or 0 for sp in specs] + [0])  # noqa: E731
+        ffs = [sp["ffn"] for sp in specs if sp["ffn"]]
+        moe = [f for f in ffs if f["kind"] == "moe"]
+        shared = [f["shared"]["ff"] for f in moe if f["shared"]]
+        return cls(name=name, arch="rumedra", vocab_size=int(js["vocab"]), hidden_size=int(js["width"]),
+                   intermediate_size=max([f["ff"] for f in ffs] + shared + [0]), num_layers=len(specs),
+                   num_heads=max(mx("heads"), mx("r_heads")), num_kv_heads=max(mx("kv_heads"), 1),
+                   head_dim=max(mx("dim"), mx("vdim"), mx("r_dim"), mx("r_vdim")), max_position=1 << 30,
+                   norm_eps=float(js["norm"]["eps"]), norm="rms", act="relu", pos_emb="rope", tie_embeddings=True,
+                   num_experts=max([f["experts"] for f in moe] + [0]),
+                   experts_per_token=max([f["top"] for f in moe] + [0]), layer_specs=specs,
+                   embed_scale=float((js.get("embedding") or {}).get("scale", 1.0)))
+
+    @classmethod
     def from_model_dir(cls, path, name: Optional[str] = None) -> "ModelConfig":
         """config.json of a model folder -> ModelConfig; the "architecture" / "model_type" key
         chooses the family."""
@@ -289,6 +316,8 @@ class ModelConfig:
             return cls.from_gevipel(js, name=name)
         if family == "vuladra":
             return cls.from_vuladra(js, name=name)
+        if family == "rumedra":
+            return cls.from_rumedra(js, name=name)
         return cls.from_hf(js, name=name)
 
     @classmethod
@@ -346,11 +375,19 @@ def layer_spec(index: int, L: dict) -> dict:
     only), norms over whole projections, an elementwise output gate; "side_by_side": windowed softmax
     attention (heads, kv_heads, dim, vdim, scale, window, left_scale) and linear attention with one constant
     decay per head (r_heads, r_dim, r_vdim, decay, right_scale) on the same input, summed;
-    "selective_scan": a gated state-space layer with a short convolution (inner, state, dt_rank, taps).
+    "selective_scan": a gated state-space layer with a short convolution (inner, state, dt_rank, taps);
+    "attention_retention": windowed softmax attention with biases, half-rotated queries and keys and an elementwise
+    output gate (heads, kv_heads, dim, vdim, scale, window, rot_dims, rot_base, rot_scaling = None or the
+    wavelength bounds, left_scale) beside rotated linear attention with one constant decay per head (r_heads, r_dim,
+    r_vdim, r_rot_dims, r_rot_base, r_rot_scaling, decay, right_scale) on the same input, summed; "hgrn": linear attention with a
+    data-dependent decay per channel whose complement is the key (r_heads, r_dim, r_vdim).
     `ffn`: None, or kind "dense" (ff) / "glu" (dense clamped GLU with biases: ff,
     limit) / "moe" (ff, limit or None for unclamped experts, experts, top, and for some stacks shared: None or
-    the always-used expert's ff and limit)."""
+    the always-used expert's ff and limit, groups: (count, kept), identity: router outputs without an expert,
+    scale: factor on the weights)."""
     m, t = L["mixer"], L["type"]
+    if t in ("attention_retention", "hgrn"):
+        return _rumedra_spec(index, t, m, L.get("mlp"))
     if t in ("pooled_attention", "side_by_side", "selective_scan"):
         return _vuladra_spec(index, t, m, L.get("mlp"))
     sp = {"index": index, "type": t, "heads": int(m["heads"]), "dim": int(m["dim"]), "vdim": int(m.get("vdim", m["dim"])),
@@ -474,7 +511,70 @@ def _vuladra_spec(index: int, t: str, m: dict, f: Optional[dict]) -> dict:
     return sp
 
 
+def _rotation(index: int, rot: Optional[dict], dim: int, pre: str = "") -> dict:
+    """Rotated dims, base and wavelength scaling of a head (absent: no rotation)."""
+    rot = rot or {}
+    sc = rot.get("scaling")
+    if sc:
+        sc = {"type": "llama3", "factor": float(sc["factor"]), "low_freq_factor": float(sc["low"]),
+              "high_freq_factor": float(sc["high"]), "original_max_position_embeddings": float(sc["original"])}
+    sp = {pre + "rot_dims": int(rot.get("dims", 0)), pre + "rot_base": float(rot.get("base", 10000.0)),
+          pre + "rot_scaling": sc or None}
+    n = sp[pre + "rot_dims"]
+    if n < 0 or n % 2 or n > dim:
+        raise ValueError(f"layer {index}: rot.dims must be even and at most the head size")
+    return sp
+
+
+def _rumedra_spec(index: int, t: str, m: dict, f: Optional[dict]) -> dict:
+    sp = {"index": index, "type": t, "kv_from": None, "maps": 1, "heads": 0, "kv_heads": 0, "dim": 0, "vdim": 0}
+    r = m
+    if t == "attention_retention":
+        left, r = m["left"], m["right"]
+        sp.update(_attention_sizes(index, left))
+        sp.update(_rotation(index, left.get("rot"), sp["dim"]))
+        sp.update(decay=[float(x) for x in r["decay"]], left_scale=float(m.get("left_scale", 1.0)),
+                  right_scale=float(m.get("right_scale", 1.0)))
+        sp.update(_rotation(index, r.get("rot"), int(r["dim"]), "r_"))
+    sp.update(r_heads=int(r["heads"]), r_dim=int(r["dim"]), r_vdim=int(r.get("vdim", r["dim"])))
+    if min(sp["r_heads"], sp["r_dim"], sp["r_vdim"]) < 1 or sp.get("pool") or \
+            ("decay" in sp and len(sp["decay"]) != sp["r_heads"]):
+        raise ValueError(f"layer {index}: bad sizes of the recurrent mixer")
+    if f is None:
+        sp["ffn"] = None
+    elif f["kind"] == "dense":
+        sp["ffn"] = {"kind": "dense", "ff": int(f["ff"])}
+    elif f["kind"] == "moe":
+        rt, sh = f["router"], f.get("shared")
+        grp = rt.get("groups") or {}
+        ff = sp["ffn"] = {"kind": "moe", "ff": int(f["expert"]["ff"]), "limit": None, "experts": int(rt["experts"]),
+                          "top": int(rt["top"]), "groups": (int(grp.get("count", 1)), int(grp.get("keep", 1))),
+                          "identity": int(rt.get("identity") or 0), "scale": float(rt.get("scale", 1.0)),
+                          "shared": {"ff": int(sh["ff"])} if sh else None}
+        n, (count, keep) = ff["experts"] + ff["identity"], ff["groups"]
+        if min(ff["experts"], count, keep) < 1 or ff["identity"] < 0 or n % count or keep > count or \
+                not 1 <= ff["top"] <= n // count * keep:
+            raise ValueError(f"layer {index}: top must be in 1..experts of the kept groups, groups of one size")
+    else:
+        raise ValueError(f"layer {index}: unknown feed-forward kind {f['kind']!r}")
+    return sp
+
+
 def layer_spec_params(h: int, sp: dict) -> int:
+    if sp["type"] in ("attention_retention", "hgrn"):
+        c, cv = sp["r_heads"] * sp["r_dim"], sp["r_heads"] * sp["r_vdim"]
+        if sp["type"] == "hgrn":
+            n = h * (2 * c + 2 * cv) + 2 * c + sp["r_vdim"]
+        else:
+            H, G, D, Dv = sp["heads"], sp["kv_heads"], sp["dim"], sp["vdim"]
+            n = (h + 1) * (H * D + G * (D + Dv)) + 2 * h * H * Dv + h * (2 * c + 3 * cv)
+        f = sp["ffn"]
+        if f and f["kind"] == "dense":
+            n += 3 * h * f["ff"]
+        elif f:
+            n += 3 * h * (f["experts"] * f["ff"] + (f["shared"]["ff"] if f["shared"] else 0)) + \
+                (f["experts"] + f["identity"]) * (h + 1)
+        return n + (2 if f else 1) * h
     if sp["type"] in ("pooled_attention", "side_by_side", "selective_scan"):
         H, G, D, Dv = sp["heads"], sp["kv_heads"], sp["dim"], sp["vdim"]
         n = h * (H * D + G * (D + Dv)) + H * Dv * h

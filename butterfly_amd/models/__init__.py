@@ -5,7 +5,9 @@ layers with a token shift over distance-biased and differential attention (model
 Gevipel, sandwich-normed layers over sloped window attention, the gated delta rule and latent
 attention with a sink, with routed plain experts (models/gevipel.py), and Vuladra, RMS-sandwiched layers
 over sigmoid attention with pooled blocks, windowed attention beside decayed linear attention, and the
-selective scan, with routed and shared clamped GLUs (models/vuladra.py)."""
+selective scan, with routed and shared clamped GLUs (models/vuladra.py), and Rumedra, pre-norm layers of
+rotated windowed attention beside retention and of linear attention with a forget gate per channel, with
+experts chosen in groups (models/rumedra.py)."""
 from .shard import LocalDims, Shard, local_dims  # noqa: F401
 from .transformer import LogicalParam, TransformerLM  # noqa: F401
 from .nesizen import NesizenLM  # noqa: F401
@@ -13,6 +15,7 @@ from .zinesun import ZinesunLM  # noqa: F401
 from .lizizen import LizizenLM  # noqa: F401
 from .gevipel import GevipelLM  # noqa: F401
 from .vuladra import VuladraLM  # noqa: F401
+from .rumedra import RumedraLM  # noqa: F401
 
 
 class LlamaForCausalLM(TransformerLM):
@@ -29,7 +32,7 @@ class GPT2LMHeadModel(TransformerLM):
 
 _ARCH = {"llama": LlamaForCausalLM, "mixtral": MixtralForCausalLM, "gpt2": GPT2LMHeadModel,
          "nesizen": NesizenLM, "zinesun": ZinesunLM, "lizizen": LizizenLM, "gevipel": GevipelLM,
-         "vuladra": VuladraLM}
+         "vuladra": VuladraLM, "rumedra": RumedraLM}
 
 
 def supports_f32(arch: str) -> bool:

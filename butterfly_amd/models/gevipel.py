@@ -111,10 +111,6 @@ class GevipelLM(PackedStack):
     # ------------------------------------------------------------------------------------
     # parameters
     # ------------------------------------------------------------------------------------
-    def _wide(self, rows: int, k: int) -> int:
-        """Rows of a projection: padded to the tuned GEMMs' 128-row tiling when its K fits them."""
-        return pad128(rows) if k % 64 == 0 else rows
-
     @staticmethod
     def _conv_channels(sp) -> int:
         return 2 * sp["kv_heads"] * sp["dim"] + sp["heads"] * sp["vdim"]

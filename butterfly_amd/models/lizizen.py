@@ -103,10 +103,6 @@ class LizizenLM(PackedStack):
     # ------------------------------------------------------------------------------------
     # parameters
     # ------------------------------------------------------------------------------------
-    def _wide(self, rows: int, k: int) -> int:
-        """Rows of a projection: padded to the tuned GEMMs' 128-row tiling when its K fits them."""
-        return pad128(rows) if k % 64 == 0 else rows
-
     def _alloc(self):
         c, W = self.cfg, self.cfg.hidden_size
         z = lambda *s: torch.zeros(*s, dtype=self.dtype, device=self.device)                  # noqa: E731

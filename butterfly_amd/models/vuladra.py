@@ -92,16 +92,6 @@ class VuladraLM(PackedStack):
     # ------------------------------------------------------------------------------------
     # parameters
     # ------------------------------------------------------------------------------------
-    def _wide(self, rows: int, k: int) -> int:
-        """Rows of a projection: padded to the tuned GEMMs' 128-row tiling when its K fits them."""
-        return pad128(rows) if k % 64 == 0 else rows
-
-    def _glu_group(self, ff: int) -> int:
-        """Row group of a GLU's [gate | up] weight: alternating 16-row blocks where the tuned GEMMs can run
-        the activation as their epilogue, else 0 (all gate rows, then all up rows)."""
-        fused = self.dtype == torch.bfloat16 and self.device.type == "cuda" and self.cfg.hidden_size % 64 == 0 and ff % 128 == 0
-        return ops.SILU_INTERLEAVE if fused else 0
-
     @staticmethod
     def _mixer_rows(sp) -> list:
         """(tensor name, rows) of the mixer's input projections in the order they are fused."""
@@ -119,14 +109,6 @@ class VuladraLM(PackedStack):
         z = lambda *s: torch.zeros(*s, dtype=self.dtype, device=self.device)                  # noqa: E731
         f = lambda *s: torch.zeros(*s, dtype=torch.float32, device=self.device)               # noqa: E731
         p = self.p
-
-        def glu(name, ff, limit, alpha, offset):
-            if self._glu_group(ff):
-                p[name + "gate_up"] = z(2 * ff, W)
-                p[name + "gate_up.b"] = ops.glu_bias_block(z(2 * ff), limit, alpha, offset)
-            else:
-                p[name + "gate_up"] = z(self._wide(2 * ff, W), W)
-            p[name + "down"] = z(self._wide(W, ff), ff)
 
         p["embed"] = z(self.dims.vocab, W)             # also the LM head; rows past the vocabulary stay zero
         for sp in self.specs:
@@ -152,13 +134,13 @@ class VuladraLM(PackedStack):
                 p[pre + "o"] = z(W, C)
             fs = sp["ffn"]
             if fs and fs["kind"] == "dense":
-                glu(pre, fs["ff"], float("inf"), 1.0, 0.0)
+                self._glu_alloc(pre, fs["ff"], float("inf"), 1.0, 0.0)
             elif fs:
                 E, F = fs["experts"], fs["ff"]
                 p[pre + "router"] = z(E, W)
                 p[pre + "experts.gate_up"], p[pre + "experts.down"] = z(E, 2 * F, W), z(E, W, F)
                 if fs["shared"]:
-                    glu(pre + "shared.", fs["shared"]["ff"], fs["shared"]["limit"], EXPERT_ALPHA, EXPERT_UP_OFFSET)
+                    self._glu_alloc(pre + "shared.", fs["shared"]["ff"], fs["shared"]["limit"], EXPERT_ALPHA, EXPERT_UP_OFFSET)
         p["final.norm"] = f(W)
 
     @property
@@ -169,23 +151,11 @@ class VuladraLM(PackedStack):
         """Checkpoint tensors by their file names ('l<i>.mix.q', 'l<i>.mlp.e<j>.up', ...), each a view into
         the fused local tensors."""
         c, p = self.cfg, self.p
-        W = c.hidden_size
         out: list[LogicalParam] = []
 
         def add(name, t, init="normal", put=None, shape=None, get=None):
             out.append(LogicalParam(name, tuple(shape or t.shape), None, 0, 0, init, get or (lambda t=t: t),
                                     put or (lambda x, t=t: t.copy_(x.reshape(t.shape)))))
-
-        def glu(name, local, ff):
-            w, grp = p[local + "gate_up"], self._glu_group(ff)
-            if grp:        # alternating blocks of `grp` gate and up rows
-                wv = w.view(ff // grp, 2, grp, W)
-                for j, n in enumerate(("gate", "up")):
-                    add(name + n, wv[:, j], shape=(ff, W), get=lambda t=wv[:, j]: t.reshape(-1, t.shape[-1]))
-            else:
-                add(name + "gate", w[:ff])
-                add(name + "up", w[ff:2 * ff])
-            add(name + "down", p[local + "down"][:W])
 
         add("embed", p["embed"][:c.vocab_size], "embed")
         for sp in self.specs:
@@ -217,7 +187,7 @@ class VuladraLM(PackedStack):
                 add(L + "mix.o", p[L + "o"])
             fs = sp["ffn"]
             if fs and fs["kind"] == "dense":
-                glu(L + "mlp.", L, fs["ff"])
+                self._glu_logical(add, L + "mlp.", L, fs["ff"])
             elif fs:
                 F = fs["ff"]
                 add(L + "mlp.router", p[L + "router"])
@@ -226,7 +196,7 @@ class VuladraLM(PackedStack):
                     add(L + f"mlp.e{e}.up", p[L + "experts.gate_up"][e, F:])
                     add(L + f"mlp.e{e}.down", p[L + "experts.down"][e])
                 if fs["shared"]:
-                    glu(L + "mlp.shared.", L + "shared.", fs["shared"]["ff"])
+                    self._glu_logical(add, L + "mlp.shared.", L + "shared.", fs["shared"]["ff"])
         add("final.norm", p["final.norm"], "ones")
         return out
 
@@ -400,11 +370,6 @@ class VuladraLM(PackedStack):
                                p[pre + "A_log"], p[pre + "dt.b"], p[pre + "D"], self.state[si + 1], meta["state_slots"],
                                meta["row_cu"], fb.positions, meta["one_row"])
         return ops.linear_act(y, p[pre + "o"])
-
-    def _glu(self, name, h, ff, limit, alpha, offset):
-        p, W = self.p, self.cfg.hidden_size
-        a = ops.linear_glu(h, p[name + "gate_up"], p.get(name + "gate_up.b"), ff, limit, alpha, offset, self._glu_group(ff))
-        return ops.linear_act(a, p[name + "down"])[:, :W]
 
     def _ffn(self, fs, pre, h):
         p = self.p

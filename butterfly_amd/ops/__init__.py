@@ -18,7 +18,7 @@ from pathlib import Path
 import torch
 
 from . import reference as ref
-from .reference import SILU_INTERLEAVE, glu_bias_block, interleave_gate_up, rope_tables, split_gate_up  # noqa: F401
+from .reference import SILU_INTERLEAVE, glu_bias_block, interleave_gate_up, rope_inv_freq, rope_tables, split_gate_up  # noqa: F401
 
 _LIB_PATH = Path(__file__).resolve().parent.parent / "_C.so"
 _loaded = False
@@ -919,13 +919,16 @@ def gla_out(o, g, norm_w, eps: float, out_dtype):
     return out
 
 
-def moe_route_scores(x, wr, top_k: int, scoring: str = "softmax", renorm: bool = True, bias=None, select_bias=None):
+def moe_route_scores(x, wr, top_k: int, scoring: str = "softmax", renorm: bool = True, bias=None, select_bias=None,
+                     groups=(1, 1), renorm_eps: float = 0.0, scale: float = 1.0):
     """Router with f32 logits -> (topk_ids [T, k] int32, topk_w [T, k] f32); scoring "softmax" |
-    "sigmoid", `renorm`: divide the chosen scores by their sum ("softmax" + renorm = the softmax
-    over the chosen logits alone); `bias` [E] f32 is added to the logits; `select_bias` [E] f32 is
-    added to the scores for the choice only, the weights being the chosen experts' plain scores."""
+    "sigmoid", `renorm`: divide the chosen scores by their sum + renorm_eps ("softmax" + renorm = the
+    softmax over the chosen logits alone); `bias` [E] f32 is added to the logits; `select_bias` [E] f32 is
+    added to the scores for the choice only, the weights being the chosen experts' plain scores.
+    groups (count, keep): E / count neighbours form a group, only members of the `keep` groups with the largest
+    choice score in them can be chosen. The weights are multiplied by `scale`."""
     if not _gpu(x):
-        return ref.moe_route_scores(x, wr, top_k, scoring, renorm, bias, select_bias)
+        return ref.moe_route_scores(x, wr, top_k, scoring, renorm, bias, select_bias, groups, renorm_eps, scale)
     T = x.shape[0]
     # logits: a GEMM with f32 accumulation and f32 output (steps of a few rows: one wave per
     # (token, expert) instead of a one-workgroup GEMM), then one wave per token picks
@@ -937,22 +940,23 @@ def moe_route_scores(x, wr, top_k: int, scoring: str = "softmax", renorm: bool =
     ids = _empty(T, top_k, dtype=torch.int32, device=x.device)
     w = _empty(T, top_k, dtype=torch.float32, device=x.device)
     torch.ops.bfly.moe_topk_scores(logits, bias, top_k, {"softmax": 0, "sigmoid": 1}[scoring], bool(renorm), ids, w,
-                                   select_bias)
+                                   select_bias, int(groups[0]), int(groups[1]), float(renorm_eps), float(scale))
     return ids, w
 
 
 def moe_glu_ffn(x, topk_ids, topk_w, gate_up_w, down_w, limit: float, alpha: float, up_offset: float = 1.0,
-                scale_input: bool = True, plain_act=None, addend=None):
+                scale_input: bool = True, plain_act=None, addend=None, identity: bool = False):
     """Routed GLU experts y = g' sigmoid(alpha g') (u' + up_offset) with g', u' clamped at `limit`
-    (inf, alpha 1, up_offset 0: the plain silu GLU). scale_input: each expert runs on (routing
+    (inf, alpha 1, up_offset 0: the plain silu GLU; alpha inf: relu(g') as the gate). scale_input: each expert runs on (routing
     score * x) and the outputs are summed; otherwise it runs on x and the sum is weighted by the
     scores. See ops.reference.moe_glu_ffn. gate_up_w [E, 2F, H], down_w [E, H, F]. plain_act
     "relu2": experts without a gate, y = relu(W_up h)^2 with gate_up_w [E, F, H] (limit, alpha and
     up_offset unused). addend [T, H] (rows may be strided): added to the f32 sum, e.g. a shared
-    expert's output."""
+    expert's output. identity (with scale_input False): ids from E on name experts without weights that
+    return x itself."""
     if not _gpu(x):
         return ref.moe_glu_ffn(x, topk_ids, topk_w, gate_up_w, down_w, limit, alpha, None, up_offset, scale_input,
-                               plain_act, addend)
+                               plain_act, addend, identity)
     T, H = x.shape
     E, F = gate_up_w.shape[0], down_w.shape[2]
     TK = T * topk_ids.shape[1]
@@ -963,7 +967,7 @@ def moe_glu_ffn(x, topk_ids, topk_w, gate_up_w, down_w, limit: float, alpha: flo
     y = _arena.get(dev, "moe_glu_y", TK * H, torch.float32)
     out = _empty(T, H, dtype=x.dtype, device=dev)
     torch.ops.bfly.moe_glu_ffn(x, topk_ids, topk_w, gate_up_w, down_w, float(limit), float(alpha), float(up_offset),
-                               bool(scale_input), work, hmid, y, out, ACTS[plain_act or "none"], addend)
+                               bool(scale_input), work, hmid, y, out, ACTS[plain_act or "none"], addend, bool(identity))
     return out
 
 
@@ -1180,7 +1184,8 @@ def diff_combine(a, lam: float, eps: float, out_mul: float, gate, Dv: int, out_d
 def glu_clamp(gu, limit: float, alpha: float, up_offset: float, group: int = 0):
     """gu [T, 2 F] = [gate | up] (rows may be a view; group > 0: alternating blocks of `group` gate
     and up columns, the layout of the GEMMs' fused gate / up epilogues): g sigmoid(alpha g) (u +
-    up_offset) with g = min(gate, limit), u = clamp(up, -limit, limit) -> [T, F]."""
+    up_offset) with g = min(gate, limit), u = clamp(up, -limit, limit) -> [T, F]. alpha = inf: relu(g) (u +
+    up_offset)."""
     if not _gpu(gu):
         return ref.glu_clamp(gu, limit, alpha, up_offset, None, group)
     out = _empty(gu.shape[0], gu.shape[1] // 2, dtype=gu.dtype, device=gu.device)
@@ -1222,12 +1227,18 @@ def post_norm_add_norm(x, y, norm_w, norm_b, eps: float, mult: float, extra, nor
     x <- x + mult * layer_norm(y; norm_w, norm_b) (+ extra [T, W] f32, e.g. the embedding output
     re-entering before a repeated span), in place in f32, and the next sublayer's input
     layer_norm(x; norm2_w, norm2_b) in out_dtype (norm2_w None: no next input, returns None). rms: RMS
-    norms with weights only in both places (the biases are None)."""
+    norms with weights only in both places (the biases are None; norm_w None: y is added as it is)."""
     if not _gpu(x):
         return ref.post_norm_add_norm(x, y, norm_w, norm_b, eps, mult, extra, norm2_w, norm2_b, out_dtype, rms)
     h = None if norm2_w is None else _empty(x.shape[0], x.shape[1], dtype=out_dtype, device=x.device)
     torch.ops.bfly.post_norm_add_norm(x, y, norm_w, norm_b, float(eps), float(mult), extra, norm2_w, norm2_b, h, bool(rms))
     return h
+
+
+def add_norm(x, y, norm_w, eps: float, out_dtype):
+    """One launch between two sublayers of a pre-norm stack: x <- x + y in place (f32), and the next sublayer's
+    input, the RMS norm of x with weight norm_w, in out_dtype (norm_w None: no next input, returns None)."""
+    return post_norm_add_norm(x, y, None, None, eps, 1.0, None, norm_w, None, out_dtype, rms=True)
 
 
 CONV_ACTS = {"none": 0, "silu": 1}
@@ -1286,8 +1297,8 @@ def delta_scan(q, k, v, b, a, a_log, dt_bias, state, state_slots, row_cu, positi
 
 
 # ---------------------------------------------------------------------------------------
-# Pooled-block attention, linear attention with a constant decay, the selective scan
-# (csrc/kernels/pooled.hip, recur.hip)
+# Pooled-block attention, linear attention with a constant decay or a forget gate per channel, the
+# selective scan (csrc/kernels/pooled.hip, recur.hip)
 # ---------------------------------------------------------------------------------------
 def pool_rows(block_size: int, pool: int) -> int:
     """Pooled rows that go with a page: the most blocks of `pool` positions that can end in one page."""
@@ -1338,17 +1349,48 @@ def decay_powers(decay, device) -> torch.Tensor:
     return torch.pow(d[:, None], torch.arange(DECAY_CHUNK + 1, dtype=torch.float64)[None]).to(torch.float32).to(device)
 
 
-def decay_scan(q, k, v, dpow, state, state_slots, row_cu, positions, act: str = "silu", one_row: bool = False):
+def decay_scan(q, k, v, dpow, state, state_slots, row_cu, positions, act: str = "silu", one_row: bool = False,
+               inv_freq=None, cs=None, k_scale: float = 1.0):
     """Linear attention with a constant decay per head over packed rows, S <- decay[h] S + k v^T, o = S^T q, the
     state pooled in `state` [slots, H, D, Dv] f32 (updated in place; a sequence whose step starts at position 0
     starts from zero). q, k [T, H, D], v [T, H, Dv] rows (views allowed), passed through `act` first; dpow =
-    decay_powers(decay). Steps of several rows per sequence run in chunks on the f32 matrix cores, steps
-    of one row (`one_row`) in place. Returns o [T, H, Dv] f32."""
+    decay_powers(decay). inv_freq [n] f32: the first 2 n dims of q and k are rotated (dimension i with i + n) by
+    positions[t] * inv_freq[i], in f32 as they are loaded (`cs`: rope_table(positions, inv_freq), when the caller
+    already has it); k is multiplied by k_scale. Steps of several rows per sequence run in chunks on the f32 matrix
+    cores, steps of one row (`one_row`) in place. Returns o [T, H, Dv] f32."""
     if not _gpu(q):
-        return ref.decay_scan(q, k, v, dpow, state, state_slots, row_cu, positions, act)
+        return ref.decay_scan(q, k, v, dpow, state, state_slots, row_cu, positions, act, inv_freq, k_scale)
+    if cs is None and inv_freq is not None:
+        cs = rope_table(positions, inv_freq)
     o = _empty(q.shape[0], q.shape[1], v.shape[2], dtype=torch.float32, device=q.device)
-    torch.ops.bfly.decay_scan(q, k, v, dpow, state, state_slots, row_cu, positions, CONV_ACTS[act], bool(one_row), o)
+    torch.ops.bfly.decay_scan(q, k, v, dpow, state, state_slots, row_cu, positions, CONV_ACTS[act], bool(one_row), o, cs,
+                              float(k_scale))
     return o
+
+
+def forget_scan(q, z, v, f_bias, lower, state, state_slots, row_cu, positions, act: str = "silu", one_row: bool = False):
+    """Linear attention whose decay per head and channel also decides what is written, over packed rows: f = lower +
+    (1 - lower) sigmoid(z + f_bias), S <- diag(f) S + (1 - f) v^T, o = S^T act(q), the state pooled as in decay_scan. q, z
+    [T, H, D], v [T, H, Dv] rows (views allowed); f_bias, lower [H * D] f32. Steps of several rows per sequence run
+    in chunks of 16 rows on the f32 matrix cores, steps of one row (`one_row`) in place. Returns o [T, H,
+    Dv] f32."""
+    if not _gpu(q):
+        return ref.forget_scan(q, z, v, f_bias, lower, state, state_slots, row_cu, positions, act)
+    o = _empty(q.shape[0], q.shape[1], v.shape[2], dtype=torch.float32, device=q.device)
+    torch.ops.bfly.forget_scan(q, z, v, f_bias, lower, state, state_slots, row_cu, positions, CONV_ACTS[act], bool(one_row), o)
+    return o
+
+
+GATE_ACTS = {"sigmoid": 0, "silu": 1}
+
+
+def head_norm_gate(o, w, eps: float, gate, mul: float, out, act: str = "silu"):
+    """out = o / sqrt(mean(o^2) + eps) * w * act(gate) * mul, the mean over each head: o [T, H, Dv] f32, w [Dv] f32 (None:
+    no weight), gate (None: no gate) and out [T, H * Dv] rows of the model's type (views allowed)."""
+    if not _gpu(o):
+        return ref.head_norm_gate(o, w, eps, gate, mul, out, act)
+    torch.ops.bfly.head_norm_gate(o, w, float(eps), gate, GATE_ACTS[act], float(mul), out)
+    return out
 
 
 def row_norm_gate(o, w, eps: float, gate, mul: float, out):

@@ -48,15 +48,14 @@ def layer_norm(x, w, b, eps, out=None, residual=None):
     return out
 
 
-def rope_tables(head_dim: int, max_pos: int, theta: float, scaling: dict | None = None,
-                device="cpu"):
-    """cos/sin tables [max_pos, head_dim/2] (f32) for the rotate-half convention.
+def rope_inv_freq(dims: int, base: float, scaling: dict | None = None) -> torch.Tensor:
+    """Angular frequencies [dims / 2] (f64) of rotary positions: base^(-2 i / dims).
 
     `scaling` supports the Llama-3.1 "llama3" frequency remap
     ({"type": "llama3", "factor", "low_freq_factor", "high_freq_factor",
       "original_max_position_embeddings"}).
     """
-    inv = 1.0 / (theta ** (torch.arange(0, head_dim, 2, dtype=torch.float64) / head_dim))
+    inv = 1.0 / (base ** (torch.arange(0, dims, 2, dtype=torch.float64) / max(dims, 1)))
     if scaling and scaling.get("type") == "llama3":
         factor = scaling["factor"]
         lo, hi = scaling["low_freq_factor"], scaling["high_freq_factor"]
@@ -66,10 +65,15 @@ def rope_tables(head_dim: int, max_pos: int, theta: float, scaling: dict | None 
         smooth = (orig / wl - lo) / (hi - lo)
         scaled = torch.where(wl > lo_wl, inv / factor, inv)
         mid = (wl <= lo_wl) & (wl >= hi_wl)
-        scaled = torch.where(mid, (1 - smooth) * inv / factor + smooth * inv, scaled)
-        inv = scaled
+        inv = torch.where(mid, (1 - smooth) * inv / factor + smooth * inv, scaled)
+    return inv
+
+
+def rope_tables(head_dim: int, max_pos: int, theta: float, scaling: dict | None = None,
+                device="cpu"):
+    """cos/sin tables [max_pos, head_dim/2] (f32) for the rotate-half convention (`scaling`: rope_inv_freq)."""
     t = torch.arange(max_pos, dtype=torch.float64)
-    f = torch.outer(t, inv)
+    f = torch.outer(t, rope_inv_freq(head_dim, theta, scaling))
     return f.cos().float().to(device), f.sin().float().to(device)
 
 
@@ -740,34 +744,40 @@ def gla_out(o, g, norm_w, eps, out_dtype):
     return (y.reshape(T, H * Dv) * F.silu(g.float())).to(out_dtype)
 
 
-def moe_route_scores(x, wr, top_k, scoring="softmax", renorm=True, bias=None, select_bias=None):
+def moe_route_scores(x, wr, top_k, scoring="softmax", renorm=True, bias=None, select_bias=None, groups=(1, 1),
+                     renorm_eps=0.0, scale=1.0):
     """Router in f32. scoring "softmax" | "sigmoid"; the top_k largest scores are chosen (ties:
-    lowest expert id); `renorm`: the chosen scores are divided by their sum (with "softmax" that
-    is the softmax over the chosen logits alone). `bias` [E] f32 is added to the logits;
+    lowest expert id); `renorm`: the chosen scores are divided by their sum + renorm_eps (with "softmax"
+    that is the softmax over the chosen logits alone). `bias` [E] f32 is added to the logits;
     `select_bias` [E] f32 is added to the scores for the choice only (the weights are the plain
-    scores of the chosen experts)."""
+    scores of the chosen experts). groups (count, keep): only members of the `keep` groups (of E / count
+    neighbours) whose best choice score is largest can be chosen. The weights are multiplied by `scale`."""
     logits = x.float() @ wr.float().t()
     if bias is not None:
         logits = logits + bias.float()
     sc = torch.softmax(logits, -1) if scoring == "softmax" else torch.sigmoid(logits)
-    if select_bias is not None:
-        ids = torch.topk(sc + select_bias.float(), top_k, -1).indices
-        w = torch.gather(sc, 1, ids)
-    else:
-        w, ids = torch.topk(sc, top_k, -1)
+    choice = sc if select_bias is None else sc + select_bias.float()
+    count, keep = groups
+    if keep < count:
+        best = choice.view(-1, count, choice.shape[1] // count).amax(-1)
+        left = torch.ones_like(best, dtype=torch.bool).scatter_(1, best.topk(keep, -1).indices, False)
+        choice = choice.masked_fill(left.repeat_interleave(choice.shape[1] // count, 1), float("-inf"))
+    ids = torch.topk(choice, top_k, -1).indices
+    w = torch.gather(sc, 1, ids)
     if renorm:
-        w = w / w.sum(-1, keepdim=True)
-    return ids.to(torch.int32), w.contiguous()
+        w = w / (w.sum(-1, keepdim=True) + renorm_eps)
+    return ids.to(torch.int32), (w * scale).contiguous()
 
 
 def moe_glu_ffn(x, topk_ids, topk_w, gate_up_w, down_w, limit, alpha, out_dtype=None, up_offset=1.0,
-                scale_input=True, plain_act=None, addend=None):
+                scale_input=True, plain_act=None, addend=None, identity=False):
     """Routed GLU experts: g = min(Wg h, limit), u = clamp(Wu h, -limit, limit),
     y = g sigmoid(alpha g) (u + up_offset), output Wd y (limit inf, alpha 1, up_offset 0: the plain
     silu GLU). scale_input: the expert runs on h = w * x and a token's expert outputs are summed;
     otherwise it runs on x and the sum is weighted by w (f32). gate_up_w [E, 2F, H] (gate rows,
     then up rows), down_w [E, H, F]. plain_act "relu2": experts without a gate, y = relu(Wu h)^2
-    with gate_up_w [E, F, H]. addend [T, H] (e.g. a shared expert's output) joins the f32 sum."""
+    with gate_up_w [E, F, H]. addend [T, H] (e.g. a shared expert's output) joins the f32 sum.
+    identity: ids from E on name experts that return x itself."""
     T, H = x.shape
     Fd = down_w.shape[2]
     out = torch.zeros(T, H, dtype=torch.float32, device=x.device)
@@ -777,6 +787,9 @@ def moe_glu_ffn(x, topk_ids, topk_w, gate_up_w, down_w, limit, alpha, out_dtype=
                 continue
             tok = (topk_ids[:, j] == e).nonzero().flatten()
             wj = topk_w[tok, j:j + 1].float()
+            if identity and e >= gate_up_w.shape[0]:
+                out[tok] += wj * x[tok].float()
+                continue
             h = (x[tok].float() * wj).to(x.dtype).float() if scale_input else x[tok].float()
             gu = h @ gate_up_w[e].float().t()
             if plain_act is not None:
@@ -785,7 +798,7 @@ def moe_glu_ffn(x, topk_ids, topk_w, gate_up_w, down_w, limit, alpha, out_dtype=
             else:
                 g = gu[:, :Fd].clamp(max=limit)
                 u = gu[:, Fd:].clamp(-limit, limit)
-                y = (g * torch.sigmoid(alpha * g) * (u + up_offset)).to(x.dtype).float()
+                y = (glu_gate(g, alpha) * (u + up_offset)).to(x.dtype).float()
             yd = y @ down_w[e].float().t()
             out[tok] += yd if scale_input else wj * yd
     if addend is not None:
@@ -1020,13 +1033,18 @@ def diff_combine(a, lam, eps, out_mul, gate, Dv, out_dtype):
     return o.to(out_dtype)
 
 
+def glu_gate(g, alpha):
+    """g sigmoid(alpha g); alpha = inf is its limit, relu(g)."""
+    return torch.relu(g) if math.isinf(alpha) else g * torch.sigmoid(alpha * g)
+
+
 def glu_clamp(gu, limit, alpha, up_offset, out_dtype=None, group=0):
     """gu [T, 2 F] = [gate | up] (group > 0: alternating blocks of `group` gate and up columns):
-    min(g, limit) sigmoid(alpha min(g, limit)) (clamp(u, +-limit) + up_offset)."""
+    glu_gate(min(g, limit), alpha) (clamp(u, +-limit) + up_offset)."""
     g, u = split_gate_up(gu, group)
     g = g.float().clamp(max=limit)
     u = u.float().clamp(min=-limit, max=limit)
-    return (g * torch.sigmoid(alpha * g) * (u + up_offset)).to(out_dtype or gu.dtype)
+    return (glu_gate(g, alpha) * (u + up_offset)).to(out_dtype or gu.dtype)
 
 
 # ---------------------------------------------------------------------------------------
@@ -1037,8 +1055,10 @@ def glu_clamp(gu, limit, alpha, up_offset, out_dtype=None, group=0):
 def post_norm_add_norm(x, y, norm_w, norm_b, eps, mult, extra, norm2_w, norm2_b, out_dtype, rms=False):
     """x <- x + mult * layer_norm(y; norm_w, norm_b) (+ extra), in place, f32; returns layer_norm(x;
     norm2_w, norm2_b) in out_dtype, the next sublayer's input (norm2_w None: nothing). rms: RMS norms
-    with weights only (the biases are None)."""
+    with weights only (the biases are None; norm_w None: y is added as it is)."""
     def norm(u, w, b):
+        if w is None:
+            return u.float()
         return _rms_offset(u.float(), w, eps, 0.0) if rms else _layer_norm_f32(u, w, b, eps)
 
     v = x + mult * norm(y, norm_w, norm_b)
@@ -1163,13 +1183,29 @@ def pool_blocks_(k_cache, v_cache, tables, row_cu, positions, slots, pool, k_poo
             v_pool[page, :, r] = v_cache[blk, :, :, j % bs].float().mean(0).to(v_pool.dtype)
 
 
-def decay_scan(q, k, v, dpow, state, state_slots, row_cu, positions, act):
+def rotate_half(x, positions, inv_freq):
+    """x [T, H, D] f32: the first 2 n dims (n = len(inv_freq)), i paired with i + n, turned by position * inv_freq[i]
+    (the f32 frequencies, product and evaluation in f64)."""
+    n = inv_freq.numel()
+    if n == 0:
+        return x
+    a = positions.double()[:, None] * inv_freq.double()[None]
+    c, s = torch.cos(a).float()[:, None, :], torch.sin(a).float()[:, None, :]
+    u, z = x[..., :n], x[..., n:2 * n]
+    return torch.cat([u * c - z * s, z * c + u * s, x[..., 2 * n:]], -1)
+
+
+def decay_scan(q, k, v, dpow, state, state_slots, row_cu, positions, act, inv_freq=None, k_scale=1.0):
     """Linear attention with a constant decay per head over packed rows, f32: q, k [T, H, D] and v [T, H,
     Dv] first pass through silu when act == "silu"; S <- dpow[h, 1] S + k v^T, o = S^T q. The state [H, D, Dv]
     of sequence s is read from state[state_slots[s]] unless its first row is at position 0 (then zero) and
-    written back after its last row. Returns o [T, H, Dv] f32."""
+    written back after its last row. inv_freq: q and k are rotated (rotate_half) after `act`; k_scale: k is
+    multiplied by it. Returns o [T, H, Dv] f32."""
     f = F.silu if act == "silu" else (lambda t: t)
     qf, kf, vf = f(q.float()), f(k.float()), f(v.float())
+    if inv_freq is not None:
+        qf, kf = rotate_half(qf, positions, inv_freq), rotate_half(kf, positions, inv_freq)
+    kf = kf * k_scale
     T, H, D = q.shape
     lam = dpow[:, 1].float()[:, None, None]
     o = torch.zeros(T, H, v.shape[2], dtype=torch.float32, device=q.device)
@@ -1183,6 +1219,42 @@ def decay_scan(q, k, v, dpow, state, state_slots, row_cu, positions, act):
             o[t] = (qf[t][:, None, :] @ S)[:, 0]
         state[sl[s]] = S
     return o
+
+
+def forget_scan(q, z, v, f_bias, lower, state, state_slots, row_cu, positions, act):
+    """Linear attention with a data-dependent decay per channel over packed rows, f32: f = lower + (1 - lower)
+    sigmoid(z + f_bias), key 1 - f: S <- diag(f) S + (1 - f) v^T, o = S^T act(q). q, z [T, H, D], v [T, H, Dv];
+    f_bias, lower [H * D] f32. The state [H, D, Dv] of sequence s is read from state[state_slots[s]] unless its first
+    row is at position 0 (then zero) and written back after its last row. Returns o [T, H, Dv] f32."""
+    T, H, D = q.shape
+    qf = F.silu(q.float()) if act == "silu" else q.float()
+    zf, lo = z.float() + f_bias.view(H, D), lower.view(H, D)
+    dec, key = lo + (1 - lo) * torch.sigmoid(zf), (1 - lo) * torch.sigmoid(-zf)
+    vf = v.float()
+    o = torch.zeros(T, H, v.shape[2], dtype=torch.float32, device=q.device)
+    cu, pos, sl = row_cu.tolist(), positions.tolist(), state_slots.tolist()
+    for s in range(len(cu) - 1):
+        if cu[s + 1] == cu[s] or sl[s] < 0:
+            continue
+        S = torch.zeros_like(state[0]) if pos[cu[s]] == 0 else state[sl[s]].clone()
+        for t in range(cu[s], cu[s + 1]):
+            S = dec[t][:, :, None] * S + key[t][:, :, None] * vf[t][:, None, :]
+            o[t] = (qf[t][:, None, :] @ S)[:, 0]
+        state[sl[s]] = S
+    return o
+
+
+def head_norm_gate(o, w, eps, gate, mul, out, act="silu"):
+    """out = o / sqrt(mean(o^2) + eps) * w * act(gate) * mul per head: o [T, H, Dv], w [Dv] or None, gate [T, H * Dv]
+    or None, act "silu" | "sigmoid"."""
+    y = o.float() * torch.rsqrt(o.float().pow(2).mean(-1, keepdim=True) + eps) * mul
+    if w is not None:
+        y = y * w.float()
+    y = y.reshape(y.shape[0], -1)
+    if gate is not None:
+        y = y * (F.silu(gate.float()) if act == "silu" else torch.sigmoid(gate.float()))
+    out.copy_(y.to(out.dtype))
+    return out
 
 
 def row_norm_gate(o, w, eps, gate, mul, out):
