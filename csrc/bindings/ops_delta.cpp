@@ -29,14 +29,15 @@ const float* opt_f32(const optional<Tensor>& t, int64_t n, const char* what) {
   return t->data_ptr<float>();
 }
 
-void post_norm_add_norm(Tensor& x, const Tensor& y, const Tensor& nw, const optional<Tensor>& nb, double eps, double mult,
+void post_norm_add_norm(Tensor& x, const Tensor& y, const optional<Tensor>& nw, const optional<Tensor>& nb, double eps, double mult,
                         const optional<Tensor>& extra, const optional<Tensor>& nw2, const optional<Tensor>& nb2,
                         const optional<Tensor>& h, bool rms) {
-  CHK_GPU(x); CHK_GPU(y); CHK_F32(x); CHK_F32(nw);
+  CHK_GPU(x); CHK_GPU(y); CHK_F32(x);
   TORCH_CHECK(x.dim() == 2 && y.dim() == 2 && y.is_contiguous() && y.sizes() == x.sizes(), "post_norm_add_norm: layouts");
   const int64_t T = x.size(0), W = x.size(1);
-  TORCH_CHECK(W >= 1 && W <= kMaxRowLds && nw.numel() == W && nb.has_value() == !rms,
+  TORCH_CHECK(W >= 1 && W <= kMaxRowLds && (nw.has_value() || rms) && nb.has_value() == !rms,
               "post_norm_add_norm: width / norm weights (biases with layer norms only)");
+  const float* w1 = opt_f32(nw, W, "post_norm_add_norm: norm weight [W]");
   const float* b1 = opt_f32(nb, W, "post_norm_add_norm: norm bias [W]");
   const float* ep = opt_f32(extra, T * W, "post_norm_add_norm: extra f32 [T, W]");
   TORCH_CHECK(nw2.has_value() == h.has_value() && nb2.has_value() == (nw2.has_value() && !rms),
@@ -49,7 +50,7 @@ void post_norm_add_norm(Tensor& x, const Tensor& y, const Tensor& nw, const opti
     TORCH_CHECK(h->is_cuda() && h->is_contiguous() && h->sizes() == x.sizes(), "post_norm_add_norm: h [T, W]");
     hp = h->data_ptr();
   }
-  bfly::launch_post_norm_add_norm(x.data_ptr<float>(), y.data_ptr(), nw.data_ptr<float>(), b1, (float)eps, (float)mult,
+  bfly::launch_post_norm_add_norm(x.data_ptr<float>(), y.data_ptr(), w1, b1, (float)eps, (float)mult,
                                   ep, w2, b2, hp, (int)T, (int)W, rms, is_f32(y), cur_stream());
 }
 
@@ -161,7 +162,7 @@ void delta_scan(const Tensor& q, const Tensor& k, const Tensor& v, const Tensor&
 }  // namespace
 
 TORCH_LIBRARY_FRAGMENT(bfly, m) {
-  m.def("post_norm_add_norm(Tensor(a!) x, Tensor y, Tensor nw, Tensor? nb, float eps, float mult, Tensor? extra, "
+  m.def("post_norm_add_norm(Tensor(a!) x, Tensor y, Tensor? nw, Tensor? nb, float eps, float mult, Tensor? extra, "
         "Tensor? nw2, Tensor? nb2, Tensor(b!)? h, bool rms=False) -> ()");
   m.def("short_conv_act(Tensor z, Tensor w, Tensor? state, Tensor? state_slots, Tensor row_cu, Tensor positions, "
         "int act, Tensor(a!) out, Tensor? bias=None) -> ()");

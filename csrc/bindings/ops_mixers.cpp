@@ -332,7 +332,8 @@ void router_logits(const Tensor& x, const Tensor& wr, Tensor& logits) {
 }
 
 void moe_topk_scores(const Tensor& logits, const optional<Tensor>& bias, int64_t top_k, int64_t scoring, bool renorm,
-                     Tensor& ids, Tensor& w, const optional<Tensor>& select_bias) {
+                     Tensor& ids, Tensor& w, const optional<Tensor>& select_bias, int64_t ngroups, int64_t keep,
+                     double renorm_eps, double scale) {
   CHK_GPU(logits); CHK_F32(logits); CHK_I32(ids); CHK_F32(w);
   const float* bp = nullptr;
   if (bias.has_value()) {
@@ -350,8 +351,11 @@ void moe_topk_scores(const Tensor& logits, const optional<Tensor>& bias, int64_t
   const int64_t T = logits.size(0), E = logits.size(1);
   TORCH_CHECK(E >= 1 && E <= 1024 && top_k >= 1 && top_k <= E, "moe_topk_scores: experts / top_k");
   TORCH_CHECK(ids.numel() == T * top_k && w.numel() == T * top_k, "moe_topk_scores: outputs");
+  TORCH_CHECK(ngroups >= 1 && keep >= 1 && keep <= ngroups && E % ngroups == 0 && top_k <= E / ngroups * keep,
+              "moe_topk_scores: groups");
   bfly::launch_moe_topk_scores(logits.data_ptr<float>(), bp, (int)top_k, (int)scoring, renorm, ids.data_ptr<int>(),
-                               w.data_ptr<float>(), (int)T, (int)E, cur_stream(), sbp);
+                               w.data_ptr<float>(), (int)T, (int)E, cur_stream(), sbp, (int)ngroups, (int)keep, (float)renorm_eps,
+                               (float)scale);
 }
 
 int64_t moe_sort_max_tiles(int64_t TK, int64_t E) { return bfly::moe_sort_max_tiles((int)TK, (int)E); }
@@ -359,7 +363,8 @@ int64_t moe_sort_max_tiles(int64_t TK, int64_t E) { return bfly::moe_sort_max_ti
 // work: int32 [TK + (E + 1) + 2 * max_tiles + 1] = perm | offsets | tiles | ntiles
 void moe_glu_ffn(const Tensor& x, const Tensor& topk_ids, const Tensor& topk_w, const Tensor& gate_up_w,
                  const Tensor& down_w, double limit, double alpha, double up_offset, bool scale_input, Tensor& work,
-                 Tensor& hmid, Tensor& y, Tensor& out, int64_t plain_act, const optional<Tensor>& addend) {
+                 Tensor& hmid, Tensor& y, Tensor& out, int64_t plain_act, const optional<Tensor>& addend,
+                 bool identity) {
   CHK_GPU(x); CHK_SAME(x, gate_up_w); CHK_SAME(x, down_w); CHK_SAME(x, hmid); CHK_SAME(x, out);
   CHK_I32(topk_ids); CHK_F32(topk_w); CHK_I32(work); CHK_F32(y);
   TORCH_CHECK(x.dim() == 2 && x.stride(1) == 1 && gate_up_w.dim() == 3 && down_w.dim() == 3 &&
@@ -384,6 +389,7 @@ void moe_glu_ffn(const Tensor& x, const Tensor& topk_ids, const Tensor& topk_w, 
     addp = addend->data_ptr();
     add_ld = addend->stride(0);
   }
+  TORCH_CHECK(!identity || !scale_input, "moe_glu_ffn: identity experts take weighted outputs");
   if (TK == 0) return;
   int* perm = work.data_ptr<int>();
   int* offsets = perm + TK;
@@ -400,7 +406,8 @@ void moe_glu_ffn(const Tensor& x, const Tensor& topk_ids, const Tensor& topk_w, 
   bfly::launch_moe_down(hmid.data_ptr(), perm, offsets, tiles, ntiles, (int)mt, down_w.data_ptr(), y.data_ptr<float>(),
                         (int)Hd, (int)F, f32, tr, s);
   bfly::launch_moe_sum(y.data_ptr<float>(), scale_input ? nullptr : topk_w.data_ptr<float>(), (int)K, out.data_ptr(),
-                       (int)T, (int)Hd, f32, s, addp, (long)add_ld);
+                       (int)T, (int)Hd, f32, s, addp, (long)add_ld, identity ? topk_ids.data_ptr<int>() : nullptr, (int)E,
+                       identity ? x.data_ptr() : nullptr, (long)x.stride(0));
 }
 
 void sample_greedy_f32(const Tensor& logits, int64_t vstart, Tensor& out_ids, Tensor& out_scores, bool check_finite) {
@@ -438,11 +445,11 @@ TORCH_LIBRARY_FRAGMENT(bfly, m) {
   m.def("gla_out(Tensor o, Tensor g, Tensor norm_w, float eps, Tensor(a!) out) -> ()");
   m.def("router_logits(Tensor x, Tensor wr, Tensor(a!) logits) -> ()");
   m.def("moe_topk_scores(Tensor logits, Tensor? bias, int top_k, int scoring, bool renorm, Tensor(a!) ids, "
-        "Tensor(b!) w, Tensor? select_bias=None) -> ()");
+        "Tensor(b!) w, Tensor? select_bias=None, int ngroups=1, int keep=1, float renorm_eps=0.0, float scale=1.0) -> ()");
   m.def("moe_sort_max_tiles(int tk, int experts) -> int", &moe_sort_max_tiles);
   m.def("moe_glu_ffn(Tensor x, Tensor topk_ids, Tensor topk_w, Tensor gate_up_w, Tensor down_w, float limit, "
         "float alpha, float up_offset, bool scale_input, Tensor(a!) work, Tensor(b!) hmid, Tensor(c!) y, "
-        "Tensor(d!) out, int plain_act=0, Tensor? addend=None) -> ()");
+        "Tensor(d!) out, int plain_act=0, Tensor? addend=None, bool identity=False) -> ()");
 }
 
 TORCH_LIBRARY_IMPL(bfly, CUDA, m) {

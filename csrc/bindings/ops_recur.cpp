@@ -1,4 +1,4 @@
-// torch.ops.bfly.* registrations of csrc/kernels/recur.hip and csrc/kernels/pooled.hip
+// torch.ops.bfly.* registrations of csrc/kernels/recur.hip, forget.hip and pooled.hip
 // (csrc/include/bfly_recur.h). Shapes, strides and index tensors are validated on the host before any launch.
 #include <ATen/ATen.h>
 #include <ATen/hip/impl/HIPStreamMasqueradingAsCUDA.h>
@@ -42,7 +42,7 @@ void check_step(const Tensor& state_slots, const Tensor& row_cu, const Tensor& p
 
 void decay_scan(const Tensor& q, const Tensor& k, const Tensor& v, const Tensor& dpow, Tensor& state,
                 const Tensor& state_slots, const Tensor& row_cu, const Tensor& positions, int64_t act, bool one_row,
-                Tensor& o) {
+                Tensor& o, const optional<Tensor>& cs, double k_scale) {
   CHK_HEADS(q); CHK_HEADS(k); CHK_HEADS(v); CHK_SAME(k, q); CHK_SAME(v, q);
   CHK_F32(dpow); CHK_F32(state); CHK_F32(o);
   const int64_t T = q.size(0), H = q.size(1), D = q.size(2), Dv = v.size(2);
@@ -54,11 +54,61 @@ void decay_scan(const Tensor& q, const Tensor& k, const Tensor& v, const Tensor&
   TORCH_CHECK(!one_row || state_slots.numel() == T, "decay_scan: one_row needs one row per sequence");
   TORCH_CHECK(act == 0 || act == 1, "decay_scan: act");
   TORCH_CHECK(D <= 8192, "decay_scan: key size");
+  const float* csp = nullptr;
+  int64_t nrot = 0;
+  if (cs.has_value()) {
+    CHK_F32(*cs);
+    TORCH_CHECK(cs->dim() == 3 && cs->size(0) == T && cs->size(1) == 2 && 2 * cs->size(2) <= D,
+                "decay_scan: cs [T, 2, n], 2 n <= D");
+    csp = cs->data_ptr<float>();
+    nrot = cs->size(2);
+  }
   TORCH_CHECK(o.dim() == 3 && o.size(0) == T && o.size(1) == H && o.size(2) == Dv, "decay_scan: o [T, H, Dv]");
   bfly::launch_decay_scan(q.data_ptr(), q.stride(0), k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0),
                           dpow.data_ptr<float>(), (int)dpow.size(1), state.data_ptr<float>(), state_slots.data_ptr<int>(),
                           row_cu.data_ptr<int>(), (int)state_slots.numel(), positions.data_ptr<int>(), (int)act,
-                          o.data_ptr<float>(), (int)T, (int)H, (int)D, (int)Dv, one_row, is_f32(q), cur_stream());
+                          csp, (int)nrot, (float)k_scale, o.data_ptr<float>(), (int)T, (int)H, (int)D, (int)Dv, one_row,
+                          is_f32(q), cur_stream());
+}
+
+void forget_scan(const Tensor& q, const Tensor& z, const Tensor& v, const Tensor& f_bias, const Tensor& lower, Tensor& state,
+                 const Tensor& state_slots, const Tensor& row_cu, const Tensor& positions, int64_t act, bool one_row,
+                 Tensor& o) {
+  CHK_HEADS(q); CHK_HEADS(z); CHK_HEADS(v); CHK_SAME(z, q); CHK_SAME(v, q);
+  CHK_F32(f_bias); CHK_F32(lower); CHK_F32(state); CHK_F32(o);
+  const int64_t T = q.size(0), H = q.size(1), D = q.size(2), Dv = v.size(2);
+  TORCH_CHECK(z.sizes() == q.sizes() && v.size(0) == T && v.size(1) == H, "forget_scan: q, z [T, H, D], v [T, H, Dv]");
+  TORCH_CHECK(f_bias.numel() == H * D && lower.numel() == H * D, "forget_scan: f_bias, lower [H * D]");
+  TORCH_CHECK(state.dim() == 4 && state.size(1) == H && state.size(2) == D && state.size(3) == Dv,
+              "forget_scan: state [slots, H, D, Dv]");
+  check_step(state_slots, row_cu, positions, T, "forget_scan");
+  TORCH_CHECK(!one_row || state_slots.numel() == T, "forget_scan: one_row needs one row per sequence");
+  TORCH_CHECK((act == 0 || act == 1) && D <= 4096, "forget_scan: act / key size");
+  TORCH_CHECK(o.dim() == 3 && o.size(0) == T && o.size(1) == H && o.size(2) == Dv, "forget_scan: o [T, H, Dv]");
+  bfly::launch_forget_scan(q.data_ptr(), q.stride(0), z.data_ptr(), z.stride(0), v.data_ptr(), v.stride(0),
+                           f_bias.data_ptr<float>(), lower.data_ptr<float>(), state.data_ptr<float>(),
+                           state_slots.data_ptr<int>(), row_cu.data_ptr<int>(), (int)state_slots.numel(),
+                           positions.data_ptr<int>(), (int)act, o.data_ptr<float>(), (int)T, (int)H, (int)D, (int)Dv, one_row,
+                           is_f32(q), cur_stream());
+}
+
+void head_norm_gate(const Tensor& o, const optional<Tensor>& w, double eps, const optional<Tensor>& gate, int64_t act,
+                    double mul, Tensor& out) {
+  CHK_F32(o); CHK_ROWS(out);
+  TORCH_CHECK(o.dim() == 3, "head_norm_gate: o [T, H, Dv]");
+  const int64_t T = o.size(0), H = o.size(1), Dv = o.size(2);
+  TORCH_CHECK(out.size(0) == T && out.size(1) == H * Dv && (act == 0 || act == 1), "head_norm_gate: out [T, H * Dv] / act");
+  const float* wp = opt_f32(w, Dv, "head_norm_gate: w f32 [Dv]");
+  const void* gp = nullptr;
+  int64_t gld = 0;
+  if (gate.has_value()) {
+    CHK_ROWS(*gate); CHK_SAME(*gate, out);
+    TORCH_CHECK(gate->sizes() == out.sizes(), "head_norm_gate: gate [T, H * Dv]");
+    gp = gate->data_ptr();
+    gld = gate->stride(0);
+  }
+  bfly::launch_head_norm_gate(o.data_ptr<float>(), wp, (float)eps, gp, gld, (int)act, (float)mul, out.data_ptr(), out.stride(0),
+                              (int)T, (int)H, (int)Dv, is_f32(out), cur_stream());
 }
 
 void row_norm_gate(const Tensor& o, const Tensor& w, double eps, const optional<Tensor>& gate, double mul, Tensor& out) {
@@ -194,7 +244,10 @@ void pool_blocks(const Tensor& k_cache, const Tensor& v_cache, const Tensor& tab
 
 TORCH_LIBRARY_FRAGMENT(bfly, m) {
   m.def("decay_scan(Tensor q, Tensor k, Tensor v, Tensor dpow, Tensor(a!) state, Tensor state_slots, Tensor row_cu, "
-        "Tensor positions, int act, bool one_row, Tensor(b!) o) -> ()");
+        "Tensor positions, int act, bool one_row, Tensor(b!) o, Tensor? cs=None, float k_scale=1.0) -> ()");
+  m.def("forget_scan(Tensor q, Tensor z, Tensor v, Tensor f_bias, Tensor lower, Tensor(a!) state, Tensor state_slots, "
+        "Tensor row_cu, Tensor positions, int act, bool one_row, Tensor(b!) o) -> ()");
+  m.def("head_norm_gate(Tensor o, Tensor? w, float eps, Tensor? gate, int act, float mul, Tensor(a!) out) -> ()");
   m.def("row_norm_gate(Tensor o, Tensor w, float eps, Tensor? gate, float mul, Tensor(a!) out) -> ()");
   m.def("selective_scan(Tensor x, Tensor dtr, Tensor b, Tensor c, Tensor z, Tensor a_log, Tensor dt_bias, Tensor d, "
         "Tensor(a!) state, Tensor state_slots, Tensor row_cu, Tensor positions, Tensor(b!) out) -> ()");
@@ -209,6 +262,8 @@ TORCH_LIBRARY_FRAGMENT(bfly, m) {
 
 TORCH_LIBRARY_IMPL(bfly, CUDA, m) {
   m.impl("decay_scan", &decay_scan);
+  m.impl("forget_scan", &forget_scan);
+  m.impl("head_norm_gate", &head_norm_gate);
   m.impl("row_norm_gate", &row_norm_gate);
   m.impl("selective_scan", &selective_scan);
   m.impl("selective_step", &selective_step);

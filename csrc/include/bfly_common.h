@@ -103,6 +103,10 @@ __device__ __forceinline__ void moe_select_topk(float logit, bool live, int lane
   }
 }
 
+// a GLU's gate g sigmoid(alpha g), whose limit for alpha = inf is relu(g) (e = exp(-alpha g), unused then)
+__device__ __forceinline__ float glu_gate(float g, float alpha, float e) {
+  return alpha < INFINITY ? g / (1.f + e) : (g < 0.f ? 0.f : g);
+}
 __device__ __forceinline__ float silu(float x) { return x / (1.f + __expf(-x)); }
 __device__ __forceinline__ float gelu_tanh(float x) {
   const float k0 = 0.7978845608028654f, k1 = 0.044715f;

@@ -10,7 +10,7 @@
 namespace bfly {
 
 // x <- x + mult * (layer_norm(y) * nw + nb) (+ extra, nullable f32 [T, W]); h (nullable) = layer_norm(x) * nw2 + nb2;
-// rms: RMS norms with weights only (nb, nb2 unused)
+// rms: RMS norms with weights only (nb, nb2 unused), nw nullable then: y is added as it is
 void launch_post_norm_add_norm(float* x, const void* y, const float* nw, const float* nb, float eps, float mult,
                                const float* extra, const float* nw2, const float* nb2, void* h, int T, int W, bool rms,
                                bool f32, hipStream_t s);

@@ -12,7 +12,8 @@ typedef __bf16 bf16;
 // EPI_SILU_GATE: the SwiGLU epilogue followed by the MoE dense decode path's routing weight
 // (what moe_gate_scale did as a separate pass): see RowScale::gate.
 // EPI_GLU: a clamped GLU with biases on gate / up rows interleaved as for EPI_SILU:
-//   Y[M, N/2] = g sigmoid(alpha g) (u + offset), g = min(gate + b_gate, limit), u = clamp(up + b_up, +-limit).
+//   Y[M, N/2] = g sigmoid(alpha g) (u + offset), g = min(gate + b_gate, limit), u = clamp(up + b_up, +-limit)
+//   (alpha = inf: relu(g) (u + offset)).
 //   `bias` then points at the epilogue's block: N bias values (bf16, interleaved like the rows)
 //   followed by the three f32 values {limit, alpha, offset} (N is even, so they are 4-byte
 //   aligned): the parameters travel with the bias, the kernels' signatures stay as they are.

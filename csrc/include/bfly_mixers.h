@@ -115,9 +115,12 @@ void launch_router_logits(const void* x, long ldx, const void* wr, float* logits
                           hipStream_t s);
 // Router choice from f32 logits [T, E] (+ bias [E], nullable): scoring 0 softmax / 1 sigmoid, top-k
 // (ties: lowest id), optional renorm. select_bias [E] (nullable) is added to the scores for the choice
-// only; the weights are the chosen experts' plain scores. E <= 1024.
+// only; the weights are the chosen experts' plain scores. keep < ngroups: only members of the `keep` groups (of
+// E / ngroups neighbours) with the largest choice score can be chosen. renorm: / (sum + renorm_eps); then times
+// scale. E <= 1024.
 void launch_moe_topk_scores(const float* logits, const float* bias, int top_k, int scoring, bool renorm, int* ids,
-                            float* w, int T, int E, hipStream_t s, const float* select_bias = nullptr);
+                            float* w, int T, int E, hipStream_t s, const float* select_bias = nullptr, int ngroups = 1,
+                            int keep = 1, float renorm_eps = 0.f, float scale = 1.f);
 // Group the T*K (token, choice) pairs by expert: perm [TK] pair indices grouped by expert,
 // offsets [E + 1], tiles [max_tiles][2] = (expert, first row) of every tile_rows-row tile, ntiles [1].
 void launch_moe_sort(const int* ids, int TK, int E, int* perm, int* offsets, int* tiles, int* ntiles, int tile_rows,
@@ -135,8 +138,10 @@ void launch_moe_glu_up(const void* x, long ldx, const float* topk_w, int K, cons
 // y[perm[r], :] = down_e(r) hmid[r]     (y f32, pair order)
 void launch_moe_down(const void* hmid, const int* perm, const int* offsets, const int* tiles, const int* ntiles,
                      int max_tiles, const void* down_w, float* y, int Hd, int F, bool f32, int tile_rows, hipStream_t s);
-// out[t] = sum_j wts[t * K + j] y[t * K + j] (+ add[t], rows of stride add_ld)   (wts == nullptr: the plain sum)
+// out[t] = sum_j wts[t * K + j] y[t * K + j] (+ add[t], rows of stride add_ld)   (wts == nullptr: the plain sum).
+// ids (nullable, with wts): where ids[t * K + j] >= E, x[t] stands in for y[t * K + j]
 void launch_moe_sum(const float* y, const float* wts, int K, void* out, int T, int Hd, bool f32, hipStream_t s,
-                    const void* add = nullptr, long add_ld = 0);
+                    const void* add = nullptr, long add_ld = 0, const int* ids = nullptr, int E = 0,
+                    const void* x = nullptr, long x_ld = 0);
 
 }  // namespace bfly

@@ -1,6 +1,6 @@
-// Host-side launch API of csrc/kernels/recur.hip and csrc/kernels/pooled.hip: linear attention with a
-// constant decay per head, the selective scan, a gated norm over whole rows, and the preparation of
-// pooled-block attention (norms over whole projections, paged append, block means). Every launcher is
+// Host-side launch API of csrc/kernels/recur.hip, forget.hip and pooled.hip: linear attention with a
+// constant decay per head or a forget gate per channel, the selective scan, gated norms over whole rows or
+// per head, and the preparation of pooled-block attention (norms over whole projections, paged append, block means). Every launcher is
 // stream-ordered, allocation-free and synchronisation-free. `f32`: the activation element type is
 // float (else bf16); norms, recurrences and their states are f32 in both.
 #pragma once
@@ -12,11 +12,24 @@ namespace bfly {
 // Linear attention with a constant decay per head over packed rows: S <- decay[h] S + k v^T, o = S^T q, q, k
 // [T, H, D] and v [T, H, Dv] rows of the activation type with row strides, first passed through silu when
 // act == 1. dpow [H, n_pow]: dpow[h][i] = decay[h]^i, n_pow >= 65. state f32 [slots, H, D, Dv], o f32
-// [T, H, Dv]. one_row: sequence s has the one row s. Sequences without a slot (-1) leave zeros.
+// [T, H, Dv]. one_row: sequence s has the one row s. Sequences without a slot (-1) leave zeros. nrot > 0: the
+// first 2 nrot dims of q and k are rotated (after act), dimension i with i + nrot, by cs [T, 2, nrot] (cosines,
+// sines); k is multiplied by k_scale.
 void launch_decay_scan(const void* q, long q_ld, const void* k, long k_ld, const void* v, long v_ld, const float* dpow,
                        int n_pow, float* state, const int* state_slots, const int* row_cu, int nseq,
-                       const int* positions, int act, float* o, int T, int H, int D, int Dv, bool one_row, bool f32,
-                       hipStream_t s);
+                       const int* positions, int act, const float* cs, int nrot, float k_scale, float* o, int T, int H,
+                       int D, int Dv, bool one_row, bool f32, hipStream_t s);
+// Linear attention with a forget gate per head and channel over packed rows: f = lower + (1 - lower) sigmoid(z +
+// f_bias), S <- diag(f) S + (1 - f) v^T, o = S^T act(q). q, z [T, H, D], v [T, H, Dv] rows of the activation type with
+// row strides; f_bias, lower f32 [H * D]; state, o, one_row as above.
+void launch_forget_scan(const void* q, long q_ld, const void* z, long z_ld, const void* v, long v_ld, const float* f_bias,
+                        const float* lower, float* state, const int* state_slots, const int* row_cu, int nseq,
+                        const int* positions, int act, float* o, int T, int H, int D, int Dv, bool one_row, bool f32,
+                        hipStream_t s);
+// out[t, h] = o[t, h] / sqrt(mean(o[t, h]^2) + eps) * w * act(gate[t, h]) * mul per head of Dv values; o f32 [T, H, Dv]
+// contiguous, w f32 [Dv] (nullable), gate (nullable; act 0 sigmoid, 1 silu) and out rows of the activation type
+void launch_head_norm_gate(const float* o, const float* w, float eps, const void* gate, long g_ld, int act, float mul,
+                           void* out, long out_ld, int T, int H, int Dv, bool f32, hipStream_t s);
 // out[t] = o[t] / sqrt(mean(o[t]^2) + eps) * w * sigmoid(gate[t]) * mul over whole rows of N values; o f32
 // contiguous, gate (nullable) and out of the activation type with row strides
 void launch_row_norm_gate(const float* o, const float* w, float eps, const void* gate, long g_ld, float mul, void* out,

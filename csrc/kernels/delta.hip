@@ -2,6 +2,7 @@
 // type (bf16 or f32; the residual, norms, decays, unit norms and the recurrent state are f32 in both):
 //   post_norm_add_norm_kernel        x <- x + mult * layer_norm(y) (+ extra), then the next sublayer's
 //                                    input layer_norm(x) with its own weight and bias
+//   add_norm_kernel                  x <- x + y, then the next sublayer's input rms_norm(x) (pre-norm stacks)
 //   short_conv_act_kernel            y_t = act(sum_j w[:, j] z_(t - taps + 1 + j)) per channel over the
 //                                    rows of a sequence (plus an optional bias); rows before the step come from the per-sequence
 //                                    history pool, zeros before position 0
@@ -95,6 +96,39 @@ __global__ __launch_bounds__(1024) void post_norm_add_norm_kernel(float* __restr
     tv o;
 #pragma unroll
     for (int e = 0; e < V; ++e) o[e] = (T)((xv[e] - mean) * rstd * wv[e] + bv[e]);
+    *reinterpret_cast<tv*>(h + t * W + c) = o;
+  }
+}
+
+// The same step of a pre-norm stack: x <- x + mult y (+ extra), h = rms_norm(x); each row is read once.
+template <typename T, int V>
+__global__ __launch_bounds__(1024) void add_norm_kernel(float* __restrict__ x, const T* __restrict__ y, float eps, float mult,
+                                                        const float* __restrict__ extra, const float* __restrict__ nw2,
+                                                        T* __restrict__ h, int W) {
+  typedef float fv __attribute__((ext_vector_type(V)));
+  typedef T tv __attribute__((ext_vector_type(V)));
+  extern __shared__ __attribute__((aligned(16))) float sy[];
+  __shared__ float red[16];
+  const long t = blockIdx.x;
+  float ss = 0.f;
+  for (int c = V * threadIdx.x; c < W; c += V * blockDim.x) {
+    const tv yv = *reinterpret_cast<const tv*>(y + t * W + c);
+    fv v = *reinterpret_cast<const fv*>(x + t * W + c);
+#pragma unroll
+    for (int e = 0; e < V; ++e) v[e] = fmaf(mult, (float)yv[e], v[e]);
+    if (extra) v += *reinterpret_cast<const fv*>(extra + t * W + c);
+    *reinterpret_cast<fv*>(x + t * W + c) = v;
+    *reinterpret_cast<fv*>(sy + c) = v;      // (read back by this thread alone)
+#pragma unroll
+    for (int e = 0; e < V; ++e) ss = fmaf(v[e], v[e], ss);
+  }
+  if (!h) return;
+  const float r = 1.f / sqrtf(block_sum(ss, red) / (float)W + eps);
+  for (int c = V * threadIdx.x; c < W; c += V * blockDim.x) {
+    const fv v = *reinterpret_cast<const fv*>(sy + c), wv = *reinterpret_cast<const fv*>(nw2 + c);
+    tv o;
+#pragma unroll
+    for (int e = 0; e < V; ++e) o[e] = (T)(v[e] * r * wv[e]);
     *reinterpret_cast<tv*>(h + t * W + c) = o;
   }
 }
@@ -451,6 +485,13 @@ void launch_post_norm_add_norm(float* x, const void* y, const float* nw, const f
                                bool f32, hipStream_t s) {
   if (T <= 0) return;
   const size_t sm = (size_t)W * sizeof(float);
+  if (!nw) {      // y as it is, one RMS norm
+#define BFLY_AN(TT, V) add_norm_kernel<TT, V><<<T, row_threads(W), sm, s>>>(x, (const TT*)y, eps, mult, extra, nw2, (TT*)h, W)
+    if (W % 4 == 0) { if (f32) BFLY_AN(float, 4); else BFLY_AN(bf16, 4); }
+    else { if (f32) BFLY_AN(float, 1); else BFLY_AN(bf16, 1); }
+#undef BFLY_AN
+    return;
+  }
 #define BFLY_PNAN(TT, V, R)                                                                                          \
   post_norm_add_norm_kernel<TT, V, R><<<T, row_threads(W), sm, s>>>(x, (const TT*)y, nw, nb, eps, mult, extra, nw2, nb2, \
                                                                     (TT*)h, W)

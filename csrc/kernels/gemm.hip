@@ -62,7 +62,7 @@ __device__ __forceinline__ GluPar glu_par(const bf16* bias, int N) {
 __device__ __forceinline__ float glu_clamped(float g, float u, const GluPar& p) {
   g = fminf(g, p.limit);
   u = fminf(fmaxf(u, -p.limit), p.limit);
-  return g / (1.f + __expf(-p.alpha * g)) * (u + p.offset);
+  return glu_gate(g, p.alpha, __expf(-p.alpha * g)) * (u + p.offset);
 }
 
 // Four consecutive output columns of one row (the tile / decode-ring accumulators hold 4

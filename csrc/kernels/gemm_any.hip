@@ -187,7 +187,7 @@ __global__ __launch_bounds__(256) void moe_glu_up_kernel(const T* __restrict__ x
       }
       const float gg = fminf(g[i][j], limit);
       const float uu = fminf(fmaxf(u[i][j], -limit), limit);
-      const float y = gg / (1.f + expf(-alpha * gg)) * (uu + up_offset);
+      const float y = glu_gate(gg, alpha, expf(-alpha * gg)) * (uu + up_offset);
       hmid[(long)r * F + c] = cvt<T>(y);
     }
   }
@@ -223,15 +223,20 @@ __global__ __launch_bounds__(256) void moe_down_kernel(const T* __restrict__ hmi
   }
 }
 
+// ids (nullable, with wts): choices from E on are identity experts, whose output is the row of x itself
 template <typename T>
 __global__ void moe_sum_kernel(const float* __restrict__ y, const float* __restrict__ wts, int Kc, T* __restrict__ out,
-                               long T_, int Hd, const T* __restrict__ add, long add_ld) {
+                               long T_, int Hd, const T* __restrict__ add, long add_ld, const int* __restrict__ ids, int E,
+                               const T* __restrict__ x, long x_ld) {
   const long n = T_ * Hd;
   for (long i = blockIdx.x * (long)blockDim.x + threadIdx.x; i < n; i += (long)gridDim.x * blockDim.x) {
     const long t = i / Hd;
     const int c = (int)(i % Hd);
     float s = 0.f;
-    if (wts) {
+    if (ids) {
+      for (int j = 0; j < Kc; ++j)
+        s = fmaf(wts[t * Kc + j], ids[t * Kc + j] >= E ? (float)x[t * x_ld + c] : y[(t * Kc + j) * Hd + c], s);
+    } else if (wts) {
       for (int j = 0; j < Kc; ++j) s = fmaf(wts[t * Kc + j], y[(t * Kc + j) * Hd + c], s);
     } else {
       for (int j = 0; j < Kc; ++j) s += y[(t * Kc + j) * Hd + c];
@@ -245,13 +250,21 @@ __global__ void moe_sum_kernel(const float* __restrict__ y, const float* __restr
 template <typename T>
 __global__ __launch_bounds__(256) void moe_sum4_kernel(const float* __restrict__ y, const float* __restrict__ wts, int Kc,
                                                        T* __restrict__ out, int Hd, const T* __restrict__ add,
-                                                       long add_ld) {
+                                                       long add_ld, const int* __restrict__ ids, int E,
+                                                       const T* __restrict__ x, long x_ld) {
   typedef T tv __attribute__((ext_vector_type(4)));
   const long t = blockIdx.x;
   for (int c = 4 * threadIdx.x; c < Hd; c += 4 * blockDim.x) {
     f32x4 s = {0.f, 0.f, 0.f, 0.f};
     for (int j = 0; j < Kc; ++j) {
-      const f32x4 v = *reinterpret_cast<const f32x4*>(y + (t * Kc + j) * Hd + c);
+      f32x4 v;
+      if (ids && ids[t * Kc + j] >= E) {
+        const tv a = *reinterpret_cast<const tv*>(x + t * x_ld + c);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] = (float)a[e];
+      } else {
+        v = *reinterpret_cast<const f32x4*>(y + (t * Kc + j) * Hd + c);
+      }
       const float w = wts ? wts[t * Kc + j] : 1.f;
 #pragma unroll
       for (int e = 0; e < 4; ++e) s[e] = fmaf(w, v[e], s[e]);
@@ -301,12 +314,14 @@ __global__ __launch_bounds__(256) void router_logits_kernel(const T* __restrict_
 }
 
 // Router choice of one token per wave from its f32 logits [E]: softmax or sigmoid scores, K rounds
-// of arg-max over the experts (ties to the lowest id).
+// of arg-max over the experts (ties to the lowest id). ngroups > keep: first the `keep` groups (of E / ngroups
+// neighbours) with the largest choice score in them are found the same way, the others' members drop out.
 __global__ __launch_bounds__(64) void moe_topk_scores_kernel(const float* __restrict__ logits,
                                                              const float* __restrict__ bias, int top_k, int scoring,
                                                              int renorm, int* __restrict__ ids, float* __restrict__ w,
-                                                             int E, const float* __restrict__ sel) {
-  __shared__ float sc[1024], raw[1024];
+                                                             int E, const float* __restrict__ sel, int ngroups, int keep,
+                                                             float renorm_eps, float scale) {
+  __shared__ float sc[1024], raw[1024], best[1024];
   const int t = blockIdx.x, lane = threadIdx.x;
   for (int e = lane; e < E; e += 64) sc[e] = logits[(long)t * E + e] + (bias ? bias[e] : 0.f);
   __syncthreads();
@@ -328,6 +343,33 @@ __global__ __launch_bounds__(64) void moe_topk_scores_kernel(const float* __rest
       raw[e] = sc[e];
       sc[e] += sel[e];
     }
+    __syncthreads();
+  }
+  if (keep < ngroups) {
+    const int gsz = E / ngroups;
+    for (int g = lane; g < ngroups; g += 64) {
+      float m = sc[g * gsz];
+      for (int e = 1; e < gsz; ++e) m = fmaxf(m, sc[g * gsz + e]);
+      best[g] = m;
+    }
+    __syncthreads();
+    for (int k = 0; k < keep; ++k) {
+      float bv = -INFINITY;
+      int bi = 0x7fffffff;
+      for (int g = lane; g < ngroups; g += 64)
+        if (best[g] > bv) { bv = best[g]; bi = g; }
+#pragma unroll
+      for (int o = 32; o > 0; o >>= 1) {
+        const float ov = __shfl_xor(bv, o, 64);
+        const int oi = __shfl_xor(bi, o, 64);
+        if (ov > bv || (ov == bv && oi < bi)) { bv = ov; bi = oi; }
+      }
+      __syncthreads();
+      if (lane == 0 && bi < ngroups) best[bi] = -INFINITY;      // kept: it leaves the race
+      __syncthreads();
+    }
+    for (int e = lane; e < E; e += 64)
+      if (best[e / gsz] != -INFINITY) sc[e] = -INFINITY;
     __syncthreads();
   }
   float sum = 0.f;
@@ -354,8 +396,10 @@ __global__ __launch_bounds__(64) void moe_topk_scores_kernel(const float* __rest
     }
     __syncthreads();
   }
-  if (renorm && lane == 0)
-    for (int k = 0; k < top_k; ++k) w[(long)t * top_k + k] /= sum;
+  if (lane == 0 && (renorm || scale != 1.f)) {
+    const float den = renorm ? sum + renorm_eps : 1.f;
+    for (int k = 0; k < top_k; ++k) w[(long)t * top_k + k] = w[(long)t * top_k + k] / den * scale;
+  }
 }
 
 // ---------------------------------------------------------------------------------------
@@ -629,7 +673,7 @@ __global__ __launch_bounds__(256) void moe_glu_up_mfma_kernel(const bf16* __rest
         if (r >= rend || c >= F) continue;
         const float gg = fminf(g[tn][tm][i], limit);
         const float uu = fminf(fmaxf(u[tn][tm][i], -limit), limit);
-        hmid[(long)r * F + c] = (bf16)(gg / (1.f + expf(-alpha * gg)) * (uu + up_offset));
+        hmid[(long)r * F + c] = (bf16)(glu_gate(gg, alpha, expf(-alpha * gg)) * (uu + up_offset));
       }
 }
 
@@ -707,9 +751,11 @@ void launch_router_logits(const void* x, long ldx, const void* wr, float* logits
 }
 
 void launch_moe_topk_scores(const float* logits, const float* bias, int top_k, int scoring, bool renorm, int* ids,
-                            float* w, int T, int E, hipStream_t s, const float* select_bias) {
+                            float* w, int T, int E, hipStream_t s, const float* select_bias, int ngroups, int keep,
+                            float renorm_eps, float scale) {
   if (T <= 0) return;
-  moe_topk_scores_kernel<<<T, 64, 0, s>>>(logits, bias, top_k, scoring, renorm, ids, w, E, select_bias);
+  moe_topk_scores_kernel<<<T, 64, 0, s>>>(logits, bias, top_k, scoring, renorm, ids, w, E, select_bias, ngroups, keep,
+                                          renorm_eps, scale);
 }
 
 int moe_sort_max_tiles(int TKp, int E) { return (TKp + 63) / 64 + E; }
@@ -762,18 +808,22 @@ void launch_moe_down(const void* hmid, const int* perm, const int* offsets, cons
 }
 
 void launch_moe_sum(const float* y, const float* wts, int K, void* out, int T, int Hd, bool f32, hipStream_t s,
-                    const void* add, long add_ld) {
+                    const void* add, long add_ld, const int* ids, int E, const void* x, long x_ld) {
   const long n = (long)T * Hd;
   if (n <= 0) return;
   const size_t al = f32 ? 16 : 8;
-  if (Hd % 4 == 0 && reinterpret_cast<uintptr_t>(out) % al == 0 && reinterpret_cast<uintptr_t>(y) % 16 == 0 &&
-      (!add || (add_ld % 4 == 0 && reinterpret_cast<uintptr_t>(add) % al == 0))) {
-    if (f32) moe_sum4_kernel<float><<<T, 256, 0, s>>>(y, wts, K, (float*)out, Hd, (const float*)add, add_ld);
-    else moe_sum4_kernel<bf16><<<T, 256, 0, s>>>(y, wts, K, (bf16*)out, Hd, (const bf16*)add, add_ld);
+  const auto rows4 = [&](const void* p, long ld) { return !p || (ld % 4 == 0 && reinterpret_cast<uintptr_t>(p) % al == 0); };
+#define BFLY_MS(TT) y, wts, K, (TT*)out, Hd, (const TT*)add, add_ld, ids, E, (const TT*)x, x_ld
+  if (Hd % 4 == 0 && rows4(out, 0) && reinterpret_cast<uintptr_t>(y) % 16 == 0 && rows4(add, add_ld) && rows4(x, x_ld)) {
+    if (f32) moe_sum4_kernel<float><<<T, 256, 0, s>>>(BFLY_MS(float));
+    else moe_sum4_kernel<bf16><<<T, 256, 0, s>>>(BFLY_MS(bf16));
     return;
   }
-  if (f32) moe_sum_kernel<float><<<ew_blocks(n), 256, 0, s>>>(y, wts, K, (float*)out, T, Hd, (const float*)add, add_ld);
-  else moe_sum_kernel<bf16><<<ew_blocks(n), 256, 0, s>>>(y, wts, K, (bf16*)out, T, Hd, (const bf16*)add, add_ld);
+#undef BFLY_MS
+#define BFLY_MS(TT) y, wts, K, (TT*)out, T, Hd, (const TT*)add, add_ld, ids, E, (const TT*)x, x_ld
+  if (f32) moe_sum_kernel<float><<<ew_blocks(n), 256, 0, s>>>(BFLY_MS(float));
+  else moe_sum_kernel<bf16><<<ew_blocks(n), 256, 0, s>>>(BFLY_MS(bf16));
+#undef BFLY_MS
 }
 
 }  // namespace bfly

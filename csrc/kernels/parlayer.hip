@@ -390,7 +390,7 @@ __global__ __launch_bounds__(256) void glu_clamp_kernel(const T* __restrict__ gu
     const int cu = group > 0 ? cg + group : F + f;
     const float g = fminf((float)gu[t * gu_ld + cg], limit);
     const float u = fminf(fmaxf((float)gu[t * gu_ld + cu], -limit), limit);
-    out[i] = (T)(g / (1.f + expf(-alpha * g)) * (u + up_offset));
+    out[i] = (T)(glu_gate(g, alpha, expf(-alpha * g)) * (u + up_offset));
   }
 }
 

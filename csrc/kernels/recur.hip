@@ -1,7 +1,8 @@
 // Recurrent mixers with pooled per-sequence state, generic in every size and in the activation type (bf16
 // or f32; decays, step sizes, states and all recurrences are f32 in both):
 //   decay_chunk_kernel, decay_step_kernel   linear attention with a constant decay per head, S <- decay S +
-//                                           k v^T, o = S^T q, in chunks on the f32 matrix cores or row by row
+//                                           k v^T, o = S^T q, in chunks on the f32 matrix cores or row by row; queries
+//                                           and keys optionally rotated by position as they are loaded
 //   selective_scan_kernel, selective_step_kernel
 //                                           S <- exp(dt A) S + dt x B, y = S C + d x, out = y silu(z), over many
 //                                           rows per sequence or one row each (with dt's projection)
@@ -10,41 +11,12 @@
 // position 0 starts from a zero state whatever its slot holds.
 #include <algorithm>
 
-#include "bfly_common.h"
 #include "bfly_recur.h"
+#include "bfly_recur_dev.h"
 
 namespace bfly {
 
 namespace {
-
-// an input's activation; FAST (bf16 inputs): hardware exp and reciprocal
-template <bool FAST>
-__device__ __forceinline__ float act_in(float v, int act) {
-  if (act != 1) return v;
-  if (FAST) return v * __builtin_amdgcn_rcpf(1.f + __expf(-v));
-  return v / (1.f + expf(-v));
-}
-
-// element 4 j .. 4 j + 3 of a row, zeros from n on
-template <typename T>
-__device__ __forceinline__ f32x4 load4(const T* __restrict__ row, int c, int n, bool vec) {
-  typedef T tv __attribute__((ext_vector_type(4)));
-  f32x4 r = {0.f, 0.f, 0.f, 0.f};
-  if (vec && c + 3 < n) {
-    const tv v = *reinterpret_cast<const tv*>(row + c);
-#pragma unroll
-    for (int e = 0; e < 4; ++e) r[e] = (float)v[e];
-  } else {
-#pragma unroll
-    for (int e = 0; e < 4; ++e)
-      if (c + e < n) r[e] = (float)row[c + e];
-  }
-  return r;
-}
-
-__device__ __forceinline__ f32x4 mfma_f32(float a, float b, f32x4 c) {
-  return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
-}
 
 // Linear attention with decay in chunks of C rows. Workgroup = (sequence, head, 64 value columns), four
 // waves of 16 columns each. With local row indices 0 .. n - 1 of a chunk and S the state before it,
@@ -56,7 +28,9 @@ __device__ __forceinline__ f32x4 mfma_f32(float a, float b, f32x4 c) {
 // tile i takes d = 16 i + 4 gg + e from group gg; q, k and the weights then come from LDS as 16-byte
 // reads. The chunk's (q . k) decay tiles at or below the diagonal are dealt to the waves and shared
 // through LDS. Rows past the sequence and dimensions past D are staged as zeros. D <= 16 NT.
-template <typename T, int NT, int C>
+// ROT: the first 2 nrot dimensions of q and k are rotated in LDS (dimension i with i + nrot) by the row's
+// cosines and sines cs[t][2][nrot]; k is multiplied by k_scale either way.
+template <typename T, int NT, int C, bool ROT>
 __global__ __launch_bounds__(256) void decay_chunk_kernel(const T* __restrict__ q, long q_ld, const T* __restrict__ k,
                                                           long k_ld, const T* __restrict__ v, long v_ld,
                                                           const float* __restrict__ dpow, int n_pow,
@@ -64,6 +38,7 @@ __global__ __launch_bounds__(256) void decay_chunk_kernel(const T* __restrict__ 
                                                           const int* __restrict__ state_slots,
                                                           const int* __restrict__ row_cu,
                                                           const int* __restrict__ positions, int act, int vec,
+                                                          const float* __restrict__ cs, int nrot, float k_scale,
                                                           float* __restrict__ o, int H, int D, int Dv) {
   constexpr int DP = 16 * NT, KP = DP + 4, VP = 68, PP = C + 4, TT = C / 16;
   extern __shared__ __attribute__((aligned(16))) float smem[];
@@ -100,6 +75,9 @@ __global__ __launch_bounds__(256) void decay_chunk_kernel(const T* __restrict__ 
   typedef T t4 __attribute__((ext_vector_type(4)));
   constexpr int NQ = (C * (DP / 4) + 255) / 256, NV = C * 16 / 256;
   t4 rq[NQ], rk[NQ], rv[NV];
+  // rotation: four pairs of a row per thread, DP / 8 threads per row; their cosines and sines travel along
+  constexpr int NR = ROT ? (C * (DP / 8) + 255) / 256 : 1;
+  f32x4 rc[NR], rs[NR];
   auto fetch4 = [&](const T* row, int c, int size, bool v4) {
     if (v4) return *reinterpret_cast<const t4*>(row + min(c, size - 4));
     t4 r;
@@ -121,12 +99,28 @@ __global__ __launch_bounds__(256) void decay_chunk_kernel(const T* __restrict__ 
       const long t = min(t0 + (i >> 4), r1 - 1);
       rv[j] = fetch4(v + t * v_ld + (long)h * Dv, c0 + 4 * (i & 15), Dv, vec & 2);
     }
+    if constexpr (ROT) {
+      if (vec & 8) {
+#pragma unroll
+        for (int j = 0; j < NR; ++j) {
+          const int i = tid + 256 * j;
+          const float* row = cs + (long)min(t0 + i / (DP / 8), r1 - 1) * 2 * nrot + min(4 * (i % (DP / 8)), nrot - 4);
+          rc[j] = *reinterpret_cast<const f32x4*>(row);
+          rs[j] = *reinterpret_cast<const f32x4*>(row + nrot);
+        }
+      }
+    }
   };
   auto stage4 = [&](const t4& r, bool row, int c, int size) {
     f32x4 a;
 #pragma unroll
     for (int e = 0; e < 4; ++e) a[e] = (row && c + e < size) ? act_in<sizeof(T) == 2>((float)r[e], act) : 0.f;
     return a;
+  };
+  auto rotate4 = [&](float* row, int i, const f32x4& c, const f32x4& sn) {      // pairs i .. i + 3
+    const f32x4 u = *reinterpret_cast<const f32x4*>(row + i), w = *reinterpret_cast<const f32x4*>(row + nrot + i);
+    *reinterpret_cast<f32x4*>(row + i) = u * c - w * sn;
+    *reinterpret_cast<f32x4*>(row + nrot + i) = w * c + u * sn;
   };
   fetch(r0);
   for (int t0 = r0; t0 < r1; t0 += C) {
@@ -136,12 +130,37 @@ __global__ __launch_bounds__(256) void decay_chunk_kernel(const T* __restrict__ 
       const int i = tid + 256 * j, t = i / (DP / 4), d = 4 * (i % (DP / 4));
       if (NQ * 256 != C * (DP / 4) && t >= C) break;
       *reinterpret_cast<f32x4*>(sq + t * KP + d) = stage4(rq[j], t < n, d, D);
-      *reinterpret_cast<f32x4*>(sk + t * KP + d) = stage4(rk[j], t < n, d, D);
+      *reinterpret_cast<f32x4*>(sk + t * KP + d) = stage4(rk[j], t < n, d, D) * k_scale;
     }
 #pragma unroll
     for (int j = 0; j < NV; ++j) {
       const int i = tid + 256 * j, t = i >> 4, c = 4 * (i & 15);
       *reinterpret_cast<f32x4*>(sv + t * VP + c) = stage4(rv[j], t < n, c0 + c, Dv);
+    }
+    if constexpr (ROT) {
+      __syncthreads();
+      if (vec & 8) {      // nrot % 4 == 0
+#pragma unroll
+        for (int j = 0; j < NR; ++j) {
+          const int i = tid + 256 * j, t = i / (DP / 8), d = 4 * (i % (DP / 8));
+          if (t < C && d < nrot) {
+            rotate4(sq + t * KP, d, rc[j], rs[j]);
+            rotate4(sk + t * KP, d, rc[j], rs[j]);
+          }
+        }
+      } else {
+        for (int i = tid; i < n * nrot; i += 256) {
+          const int t = i / nrot, d = i - t * nrot;
+          const float c = cs[(long)(t0 + t) * 2 * nrot + d], sn = cs[(long)(t0 + t) * 2 * nrot + nrot + d];
+          float* qr = sq + t * KP + d;
+          float* kr = sk + t * KP + d;
+          const float qu = qr[0], qw = qr[nrot], ku = kr[0], kw = kr[nrot];
+          qr[0] = qu * c - qw * sn;
+          qr[nrot] = qw * c + qu * sn;
+          kr[0] = ku * c - kw * sn;
+          kr[nrot] = kw * c + ku * sn;
+        }
+      }
     }
     if (t0 + C < r1) fetch(t0 + C);      // in flight during the products below
     __syncthreads();
@@ -238,6 +257,7 @@ __global__ __launch_bounds__(256) void decay_step_kernel(const T* __restrict__ q
                                                          float* __restrict__ state, const int* __restrict__ state_slots,
                                                          const int* __restrict__ row_cu,
                                                          const int* __restrict__ positions, int act, int vec,
+                                                         const float* __restrict__ cs, int nrot, float k_scale,
                                                          float* __restrict__ o, int H, int D, int Dv) {
   extern __shared__ __attribute__((aligned(16))) float smem[];
   float* sq = smem;            // [D]
@@ -256,9 +276,20 @@ __global__ __launch_bounds__(256) void decay_step_kernel(const T* __restrict__ q
   float* S = state + ((long)slot * H + h) * D * Dv;
   const bool sv4 = (vec & 4) && c + 3 < Dv;      // 16-byte state rows
   for (int t = r0; t < r1; ++t) {
+    const T* qr = q + (long)t * q_ld + (long)h * D;
+    const T* kr = k + (long)t * k_ld + (long)h * D;
     for (int d = tid; d < D; d += 256) {
-      sq[d] = act_in<sizeof(T) == 2>((float)q[(long)t * q_ld + (long)h * D + d], act);
-      sk[d] = act_in<sizeof(T) == 2>((float)k[(long)t * k_ld + (long)h * D + d], act);
+      float qv = act_in<sizeof(T) == 2>((float)qr[d], act), kv = act_in<sizeof(T) == 2>((float)kr[d], act);
+      if (d < 2 * nrot) {      // rotated with its partner: (u c - w s, w c + u s)
+        const bool hi = d >= nrot;
+        const int i = hi ? d - nrot : d, m = hi ? i : d + nrot;
+        const float c = cs[(long)t * 2 * nrot + i], sn = cs[(long)t * 2 * nrot + nrot + i];
+        const float qm = act_in<sizeof(T) == 2>((float)qr[m], act), km = act_in<sizeof(T) == 2>((float)kr[m], act);
+        qv = hi ? qv * c + qm * sn : qv * c - qm * sn;
+        kv = hi ? kv * c + km * sn : kv * c - km * sn;
+      }
+      sq[d] = qv;
+      sk[d] = kv * k_scale;
     }
     f32x4 vv = load4(v + (long)t * v_ld + (long)h * Dv, c, Dv, vec & 2);
 #pragma unroll
@@ -299,13 +330,6 @@ __global__ __launch_bounds__(256) void decay_step_kernel(const T* __restrict__ q
     }
     __syncthreads();
   }
-}
-
-// sum over the four lanes of a quad, in every lane
-__device__ __forceinline__ float quad_sum(float v) {
-  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0xB1, 0xF, 0xF, true));
-  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x4E, 0xF, 0xF, true));
-  return v;
 }
 
 // softplus, silu and exp(dt A) of the selective scan. FAST (bf16 activations): the hardware exp / log /
@@ -574,51 +598,53 @@ __global__ __launch_bounds__(256) void row_norm_gate_kernel(const float* __restr
   }
 }
 
-bool rows_aligned(const void* p, long ld, size_t esz) {
-  return ld % 4 == 0 && reinterpret_cast<uintptr_t>(p) % (4 * esz) == 0;
-}
-
-template <typename T, int NT, int C>
+template <typename T, int NT, int C, bool ROT>
 void decay_chunk_launch(const T* q, long q_ld, const T* k, long k_ld, const T* v, long v_ld, const float* dpow, int n_pow,
                         float* state, const int* state_slots, const int* row_cu, int nseq, const int* positions, int act,
-                        int vec, float* o, int H, int D, int Dv, hipStream_t s) {
+                        int vec, const float* cs, int nrot, float k_scale, float* o, int H, int D, int Dv, hipStream_t s) {
   constexpr size_t lds = (size_t)(2 * C * (16 * NT + 4) + C * 68 + C * (C + 4) + C + 1) * sizeof(float);
   static bool once = false;
   if (!once) {
-    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&decay_chunk_kernel<T, NT, C>),
+    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&decay_chunk_kernel<T, NT, C, ROT>),
                               hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     once = true;
   }
   dim3 grid(nseq, H, (Dv + 63) / 64);
-  decay_chunk_kernel<T, NT, C><<<grid, 256, lds, s>>>(q, q_ld, k, k_ld, v, v_ld, dpow, n_pow, state, state_slots, row_cu,
-                                                      positions, act, vec, o, H, D, Dv);
+  decay_chunk_kernel<T, NT, C, ROT><<<grid, 256, lds, s>>>(q, q_ld, k, k_ld, v, v_ld, dpow, n_pow, state, state_slots,
+                                                           row_cu, positions, act, vec, cs, nrot, k_scale, o, H, D, Dv);
 }
 
 template <typename T>
 void decay_scan_t(const T* q, long q_ld, const T* k, long k_ld, const T* v, long v_ld, const float* dpow, int n_pow,
                   float* state, const int* state_slots, const int* row_cu, int nseq, const int* positions, int act,
-                  float* o, int H, int D, int Dv, bool one_row, hipStream_t s) {
-  int vec = 0;      // 1: q and k rows, 2: v rows, 4: state rows in four-element accesses
+                  const float* cs, int nrot, float k_scale, float* o, int H, int D, int Dv, bool one_row, hipStream_t s) {
+  int vec = 0;      // 1: q and k rows, 2: v rows, 4: state rows, 8: rotated pairs in four-element accesses
   if (D % 4 == 0 && rows_aligned(q, q_ld, sizeof(T)) && rows_aligned(k, k_ld, sizeof(T))) vec |= 1;
   if (Dv % 4 == 0 && rows_aligned(v, v_ld, sizeof(T))) vec |= 2;
   if (Dv % 4 == 0) vec |= 4;
+  if (nrot > 0 && nrot % 4 == 0 && rows_aligned(cs, 2 * nrot, sizeof(float))) vec |= 8;
   if (one_row || D > 256) {
     dim3 grid(nseq, H, (Dv + 63) / 64);
     decay_step_kernel<T><<<grid, 256, 2 * (size_t)D * sizeof(float), s>>>(
-        q, q_ld, k, k_ld, v, v_ld, dpow, n_pow, state, state_slots, one_row ? nullptr : row_cu, positions, act, vec, o, H, D,
-        Dv);
+        q, q_ld, k, k_ld, v, v_ld, dpow, n_pow, state, state_slots, one_row ? nullptr : row_cu, positions, act, vec, cs, nrot,
+        k_scale, o, H, D, Dv);
     return;
   }
-#define BFLY_DCH(NT, C)                                                                                              \
-  decay_chunk_launch<T, NT, C>(q, q_ld, k, k_ld, v, v_ld, dpow, n_pow, state, state_slots, row_cu, nseq, positions, act, \
-                               vec, o, H, D, Dv, s)
-  if (D <= 32) BFLY_DCH(2, 64);
-  else if (D <= 64) BFLY_DCH(4, 64);
-  else if (D <= 96) BFLY_DCH(6, 64);
-  else if (D <= 128) BFLY_DCH(8, 64);
-  else if (D <= 192) BFLY_DCH(12, 32);
-  else BFLY_DCH(16, 32);
+#define BFLY_DCH2(NT, C, ROT)                                                                                          \
+  decay_chunk_launch<T, NT, C, ROT>(q, q_ld, k, k_ld, v, v_ld, dpow, n_pow, state, state_slots, row_cu, nseq, positions, \
+                                    act, vec, cs, nrot, k_scale, o, H, D, Dv, s)
+#define BFLY_DCH(NT, C)                                                 \
+  {                                                                     \
+    if (nrot > 0) BFLY_DCH2(NT, C, true); else BFLY_DCH2(NT, C, false); \
+  }
+  if (D <= 32) BFLY_DCH(2, 64)
+  else if (D <= 64) BFLY_DCH(4, 64)
+  else if (D <= 96) BFLY_DCH(6, 64)
+  else if (D <= 128) BFLY_DCH(8, 64)
+  else if (D <= 192) BFLY_DCH(12, 32)
+  else BFLY_DCH(16, 32)
 #undef BFLY_DCH
+#undef BFLY_DCH2
 }
 
 template <typename T>
@@ -668,15 +694,15 @@ int selective_scan_t(const T* x, long x_ld, const float* dtr, long dt_ld, const 
 
 void launch_decay_scan(const void* q, long q_ld, const void* k, long k_ld, const void* v, long v_ld, const float* dpow,
                        int n_pow, float* state, const int* state_slots, const int* row_cu, int nseq,
-                       const int* positions, int act, float* o, int T, int H, int D, int Dv, bool one_row, bool f32,
-                       hipStream_t s) {
+                       const int* positions, int act, const float* cs, int nrot, float k_scale, float* o, int T, int H,
+                       int D, int Dv, bool one_row, bool f32, hipStream_t s) {
   if (T <= 0 || nseq <= 0) return;
   if (f32)
     decay_scan_t<float>((const float*)q, q_ld, (const float*)k, k_ld, (const float*)v, v_ld, dpow, n_pow, state,
-                        state_slots, row_cu, nseq, positions, act, o, H, D, Dv, one_row, s);
+                        state_slots, row_cu, nseq, positions, act, cs, nrot, k_scale, o, H, D, Dv, one_row, s);
   else
     decay_scan_t<bf16>((const bf16*)q, q_ld, (const bf16*)k, k_ld, (const bf16*)v, v_ld, dpow, n_pow, state, state_slots,
-                       row_cu, nseq, positions, act, o, H, D, Dv, one_row, s);
+                       row_cu, nseq, positions, act, cs, nrot, k_scale, o, H, D, Dv, one_row, s);
 }
 
 void launch_row_norm_gate(const float* o, const float* w, float eps, const void* gate, long g_ld, float mul, void* out,
