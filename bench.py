@@ -92,7 +92,7 @@ def build_parser() -> argparse.ArgumentParser:
                     help="single-stage layouts: host waits for each step's tokens before scheduling the "
                          "next (default: EngineConfig.async_decode, the next step overlaps the host work)")
     ap.add_argument("--out", default=None, help="also write the JSON line here")
-    ap.add_argument("--mixer-family", default="nesizen", choices=["nesizen", "zinesun", "lizizen", "gevipel", "vuladra"],
+    ap.add_argument("--mixer-family", default="nesizen", choices=["nesizen", "zinesun", "lizizen", "gevipel", "vuladra", "rumedra"],
                     help="with --mixer-compare: the heterogeneous family that is timed (nesizen: beside a Mixtral "
                          "stack; zinesun: latent attention beside a Nesizen stack of plain windowed attention; "
                          "lizizen: parallel layers of distance-biased and differential attention with dense GLU "
@@ -102,7 +102,10 @@ def build_parser() -> argparse.ArgumentParser:
                          "attention and gated linear attention over routed GLU experts; "
                          "vuladra: windowed attention beside decayed linear attention, the selective scan and sigmoid "
                          "attention with pooled blocks over dense and routed GLUs with a shared expert beside a Nesizen "
-                         "stack of windowed attention and gated linear attention)")
+                         "stack of windowed attention and gated linear attention; "
+                         "rumedra: windowed attention beside retention and linear attention with a forget gate per "
+                         "channel over dense ReLU GLUs and grouped routed experts with a shared one, beside the same "
+                         "kind of Nesizen stack)")
     ap.add_argument("--mixer-compare", default=None, metavar="SIZES",
                     help="instead of the headline run: prefill and decode throughput of a Nesizen stack "
                          "(windowed attention, shared keys, gated linear attention, sigmoid MoE) beside a "
@@ -284,6 +287,37 @@ def run_mixer_compare(a) -> int:
                                                  {"type": "attention", "mixer": plain, "mlp": moe},
                                                  {"type": "gla", "mixer": gla, "mlp": moe}]}, name=f"nesizen-scan-{size}")
             pair = (vul, nes5)
+        if a.mixer_family == "rumedra":
+            # gated windowed attention beside retention (half the heads each), linear attention with a forget gate
+            # per channel, one dense ReLU GLU (two thirds of the width: the parameters of the counterpart's two
+            # matrices), silu GLU experts in two groups of which one is kept, with a shared expert (one routed choice
+            # less: the same active FLOPs); beside windowed GQA attention and gated linear attention of the same heads
+            # and window, one stream
+            w2 = win // 2
+            par = {"left": {"heads": H // 2, "kv_heads": max(G // 2, 1), "dim": D, "vdim": D, "scale": D ** -0.5,
+                            "mask": {"size": w2}, "rot": {"dims": D // 2, "base": 5e5, "scaling": {
+                                "factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}},
+                   "right": {"heads": H // 2, "dim": D, "vdim": D, "rot": {"dims": D, "base": 1e4},
+                             "decay": [1.0 - 2.0 ** (-3 - 5 * i / (H // 2)) for i in range(H // 2)]},
+                   "left_scale": 0.9, "right_scale": 0.8}
+            hgr = {"heads": H, "dim": D, "vdim": D}
+            rmoe = {"kind": "moe", "expert": {"ff": eff}, "shared": {"ff": eff},
+                    "router": {"experts": E, "top": top - 1, "groups": {"count": 2, "keep": 1}, "identity": 0, "scale": 1.5}}
+            rum = ModelConfig.from_rumedra({"architecture": "Rumedra", "vocab": 32000, "width": W, "norm": {"eps": 1e-6},
+                                            "embedding": {"scale": 1.0}, "layers": [
+                                                {"type": "parallel", "mixer": par,
+                                                 "mlp": {"kind": "dense", "ff": 2 * dff // 3 // 128 * 128}},
+                                                {"type": "hgrn2", "mixer": hgr, "mlp": rmoe},
+                                                {"type": "parallel", "mixer": par, "mlp": rmoe},
+                                                {"type": "hgrn2", "mixer": hgr, "mlp": rmoe}]}, name=f"rumedra-{size}")
+            plain = dict(attn, mask={"size": w2, "keep_first": 0})
+            nes6 = ModelConfig.from_nesizen({"architecture": "Nesizen", "vocab": 32000, "width": W, "streams": 1,
+                                             "norm": {"eps": 1e-6}, "layers": [
+                                                 {"type": "attention", "mixer": plain, "mlp": {"kind": "dense", "ff": dff}},
+                                                 {"type": "gla", "mixer": gla, "mlp": moe},
+                                                 {"type": "attention", "mixer": plain, "mlp": moe},
+                                                 {"type": "gla", "mixer": gla, "mlp": moe}]}, name=f"nesizen-gla-{size}")
+            pair = (rum, nes6)
         for cfg in pair:
             ecfg = EngineConfig(max_batch=B, max_seq_len=P + K + Wm + 8, max_prefill_tokens=8192,
                                 kv_cache_tokens=B * (P + K + Wm + 40), use_graphs=not a.no_graphs,

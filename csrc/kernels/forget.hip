@@ -7,6 +7,7 @@
 // Rows of a step are packed: sequence s owns rows row_cu[s] .. row_cu[s+1]; a sequence whose first row is at
 // position 0 starts from a zero state whatever its slot holds.
 #include <algorithm>
+#include <type_traits>
 
 #include "bfly_recur.h"
 #include "bfly_recur_dev.h"
@@ -22,6 +23,17 @@ __device__ __forceinline__ void sigmoid2(float x, float& s, float& c) {
   const float r = FAST ? __builtin_amdgcn_rcpf(1.f + e) : 1.f / (1.f + e);
   s = x < 0.f ? e * r : r;
   c = x < 0.f ? r : e * r;
+}
+
+// One element at a vector plus a scalar byte offset from a uniform base. (The rows of one chunk; callers clamp row and
+// channel to the tensor.)
+__device__ __forceinline__ __amdgpu_buffer_rsrc_t rows_rsrc(const void* base) {
+  return __builtin_amdgcn_make_buffer_rsrc(const_cast<void*>(base), (short)0, 0x7fffffff, 0x00027000);
+}
+template <typename T>
+__device__ __forceinline__ T row_load(__amdgpu_buffer_rsrc_t r, int voff, int soff) {
+  if constexpr (sizeof(T) == 2) return __builtin_bit_cast(T, __builtin_amdgcn_raw_buffer_load_b16(r, voff, soff, 0));
+  else return __builtin_bit_cast(T, __builtin_amdgcn_raw_buffer_load_b32(r, voff, soff, 0));
 }
 
 // Chunks of 16 rows. Workgroup = (sequence, head, 64 value columns), four waves of 16 columns each. With F_t = f_0 .. f_t
@@ -56,7 +68,7 @@ __global__ __launch_bounds__(256) void forget_chunk_kernel(const T* __restrict__
   float* sp = sv + C * VP;              // [C][PP]
   float* sl = sp + C * PP;              // [DP] F of the last row
   const int s = blockIdx.x, h = blockIdx.y, c0 = blockIdx.z * 64;
-  const int r0 = row_cu[s], r1 = row_cu[s + 1];
+  const int r0 = __builtin_amdgcn_readfirstlane(row_cu[s]), r1 = __builtin_amdgcn_readfirstlane(row_cu[s + 1]);
   if (r1 <= r0) return;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, m = lane & 15, gg = lane >> 4;
   const int slot = state_slots[s];
@@ -99,18 +111,22 @@ __global__ __launch_bounds__(256) void forget_chunk_kernel(const T* __restrict__
   T rq[NI][C], rz[NI][C];
   t4 rv;
   auto fetch = [&](int t0) {
+    // (one descriptor per chunk; a load takes the channel's vector offset and the row's scalar offset)
+    const __amdgpu_buffer_rsrc_t qb = rows_rsrc(q + (long)t0 * q_ld + (long)h * D);
+    const __amdgpu_buffer_rsrc_t zb = rows_rsrc(z + (long)t0 * z_ld + (long)h * D);
+    const int qs = (int)q_ld * (int)sizeof(T), zs = (int)z_ld * (int)sizeof(T);
+    const int last = r1 - 1 - t0;
 #pragma unroll
     for (int u = 0; u < NI; ++u) {
-      const int idx = tid + 256 * u, d = min(idx < DP ? idx : idx - DP, D - 1);
+      const int idx = tid + 256 * u;
+      const int d = min(idx < DP ? idx : idx - DP, D - 1) * (int)sizeof(T);
       if (idx < DP) {
-        const T* qc = q + (long)h * D + d;
 #pragma unroll
-        for (int i = 0; i < C; ++i) rq[u][i] = qc[(long)min(t0 + i, r1 - 1) * q_ld];
+        for (int i = 0; i < C; ++i) rq[u][i] = row_load<T>(qb, d, __builtin_amdgcn_readfirstlane(min(i, last) * qs));
       }
-      if (idx < 2 * DP) {
-        const T* zc = z + (long)h * D + d;
+      if (NI * 256 == 2 * DP || idx < 2 * DP) {
 #pragma unroll
-        for (int i = 0; i < C; ++i) rz[u][i] = zc[(long)min(t0 + i, r1 - 1) * z_ld];
+        for (int i = 0; i < C; ++i) rz[u][i] = row_load<T>(zb, d, __builtin_amdgcn_readfirstlane(min(i, last) * zs));
       }
     }
     const T* vr = v + (long)min(t0 + (tid >> 4), r1 - 1) * v_ld + (long)h * Dv;
@@ -122,41 +138,57 @@ __global__ __launch_bounds__(256) void forget_chunk_kernel(const T* __restrict__
       for (int e = 0; e < 4; ++e) rv[e] = vr[min(c + e, Dv - 1)];
     }
   };
-  fetch(r0);
-  for (int t0 = r0; t0 < r1; t0 += C) {
-    const int n = min(C, r1 - t0);
+  // Gates of this thread's channels into LDS. No branch: a row past the sequence is set to f = 1, k = q = 0 by factors
+  // (`tail`: the last chunk has such rows), a channel past D has q = 0 (its state row is never read or stored).
+  auto stage = [&](int n, auto tail) {
 #pragma unroll
     for (int u = 0; u < NI; ++u) {
       const int idx = tid + 256 * u;
+      const float one = 1.f - rl[u];
       if (idx < DP) {
+        const float qm = idx < D ? 1.f : 0.f;
         float F = 1.f;
 #pragma unroll
         for (int i = 0; i < C; ++i) {
-          const bool in = i < n && idx < D;
+          const float in = decltype(tail)::value ? (i < n ? 1.f : 0.f) : 1.f;
           float sg, cg;
           sigmoid2<FAST>((float)rz[u][i] + rb[u], sg, cg);
-          const float f = in ? rl[u] + (1.f - rl[u]) * sg : 1.f, qv = in ? act_in<FAST>((float)rq[u][i], act) : 0.f;
+          float f = fmaf(one, sg, rl[u]), qv = act_in<FAST>((float)rq[u][i], act) * qm;
+          if (decltype(tail)::value) {
+            f = fmaf(in, f, 1.f - in);
+            qv *= in;
+          }
           F *= f;
           sq[i * KP + idx] = qv;
           sf[i * KP + idx] = f;
           sqf[i * KP + idx] = qv * F;
         }
         sl[idx] = F;
-      } else if (idx < 2 * DP) {
+      } else if (NI * 256 == 2 * DP || idx < 2 * DP) {
         const int d = idx - DP;
         float B = 1.f;
 #pragma unroll
         for (int i = C - 1; i >= 0; --i) {
-          const bool in = i < n && d < D;
+          const float in = decltype(tail)::value ? (i < n ? 1.f : 0.f) : 1.f;
           float sg, cg;
           sigmoid2<FAST>((float)rz[u][i] + rb[u], sg, cg);
-          const float k = in ? (1.f - rl[u]) * cg : 0.f;
+          float f = fmaf(one, sg, rl[u]), k = one * cg;
+          if (decltype(tail)::value) {
+            f = fmaf(in, f, 1.f - in);
+            k *= in;
+          }
           sk[i * KP + d] = k;
           skb[i * KP + d] = k * B;
-          B *= in ? rl[u] + (1.f - rl[u]) * sg : 1.f;
+          B *= f;
         }
       }
     }
+  };
+  fetch(r0);
+  for (int t0 = r0; t0 < r1; t0 += C) {
+    const int n = min(C, r1 - t0);
+    if (n == C) stage(n, std::false_type{});
+    else stage(n, std::true_type{});
     {
       const int t = tid >> 4, c = 4 * (tid & 15);
       f32x4 a;
@@ -227,13 +259,15 @@ __global__ __launch_bounds__(256) void forget_chunk_kernel(const T* __restrict__
     // (the next chunk's staging writes nothing that is read after the barrier above but sp, which is rewritten only
     // after its own first barrier)
   }
+  int De = D;
+  asm volatile("" : "+s"(De));      // (the bounds are compared anew: kept masks would fill the scalar registers)
   if (live) {
 #pragma unroll
     for (int i = 0; i < NT; ++i)
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         const int d = 16 * i + 4 * gg + e;
-        if (d < D) S[(long)d * Dv] = st[i][e];
+        if (d < De) S[(long)d * Dv] = st[i][e];
       }
   }
 }
