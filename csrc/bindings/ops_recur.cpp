@@ -84,6 +84,7 @@ void forget_scan(const Tensor& q, const Tensor& z, const Tensor& v, const Tensor
   check_step(state_slots, row_cu, positions, T, "forget_scan");
   TORCH_CHECK(!one_row || state_slots.numel() == T, "forget_scan: one_row needs one row per sequence");
   TORCH_CHECK((act == 0 || act == 1) && D <= 4096, "forget_scan: act / key size");
+  TORCH_CHECK(q.stride(0) < (1 << 21) && z.stride(0) < (1 << 21), "forget_scan: row strides");      // (24-bit byte offsets)
   TORCH_CHECK(o.dim() == 3 && o.size(0) == T && o.size(1) == H && o.size(2) == Dv, "forget_scan: o [T, H, Dv]");
   bfly::launch_forget_scan(q.data_ptr(), q.stride(0), z.data_ptr(), z.stride(0), v.data_ptr(), v.stride(0),
                            f_bias.data_ptr<float>(), lower.data_ptr<float>(), state.data_ptr<float>(),

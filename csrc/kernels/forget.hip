@@ -25,29 +25,38 @@ __device__ __forceinline__ void sigmoid2(float x, float& s, float& c) {
   c = x < 0.f ? r : e * r;
 }
 
-// One element at a vector plus a scalar byte offset from a uniform base. (The rows of one chunk; callers clamp row and
-// channel to the tensor.)
+// One element at a byte offset below 2^31 from a uniform base. (Rows of one chunk; callers clamp row and channel to the
+// tensor.)
 __device__ __forceinline__ __amdgpu_buffer_rsrc_t rows_rsrc(const void* base) {
   return __builtin_amdgcn_make_buffer_rsrc(const_cast<void*>(base), (short)0, 0x7fffffff, 0x00027000);
 }
 template <typename T>
-__device__ __forceinline__ T row_load(__amdgpu_buffer_rsrc_t r, int voff, int soff) {
-  if constexpr (sizeof(T) == 2) return __builtin_bit_cast(T, __builtin_amdgcn_raw_buffer_load_b16(r, voff, soff, 0));
-  else return __builtin_bit_cast(T, __builtin_amdgcn_raw_buffer_load_b32(r, voff, soff, 0));
+__device__ __forceinline__ T row_load(__amdgpu_buffer_rsrc_t r, int off) {
+  if constexpr (sizeof(T) == 2) return __builtin_bit_cast(T, __builtin_amdgcn_raw_buffer_load_b16(r, off, 0, 0));
+  else return __builtin_bit_cast(T, __builtin_amdgcn_raw_buffer_load_b32(r, off, 0, 0));
 }
 
-// Chunks of 16 rows. Workgroup = (sequence, head, 64 value columns), four waves of 16 columns each. With F_t = f_0 .. f_t
-// and B_j = f_(j+1) .. f_(n-1) (products per channel over the chunk's rows) and S the state before it,
+// sum over the 32 lanes of a half wave, in its upper sixteen lanes
+__device__ __forceinline__ float half_sum(float v) {
+  v = row16_sum(v);
+  return v + __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x142, 0xA, 0xF, false));
+}
+
+// Chunks of 16 rows. Workgroup = (sequence, head, 64 value columns), eight waves: wave & 3 names 16 columns, wave >> 2 a half
+// of the state's rows. With F_t = f_0 .. f_t and B_j = f_(j+1) .. f_(n-1) (products per channel over the chunk's rows)
+// and S the state before it,
 //   o_t = (q_t F_t) S + sum_(j <= t) (sum_d q_td k_jd f_(j+1)d .. f_td) v_j,      S <- diag(F_(n-1)) S + sum_j (k_j B_j) v_j^T
 // with k = 1 - f. Only products of decays occur, never quotients, so gates of any size are safe. The inputs of one
-// channel's 16 rows are held by one thread, which forms the running products on the way into LDS: the first DP of
-// 2 DP roles stage q, f and q F, the others k and k B. The products with the state and with v run on the f32 matrix
-// cores (16x16x4 tiles); a wave keeps its columns' state in the accumulator layout (tile i, element e: row d = 16 i
-// + 4 gg + e of lane group gg), which is also the B operand of (q F) S. The 16 x 16 weights of the second sum
-// are formed on the vector units while the matrix cores are busy: 16 lanes per row t share its channels, and q_t times
-// the decays so far is carried down j. Rows past the sequence have f = 1, k = q = 0. D <= 16 NT.
+// channel are held by two lanes of a wave, eight rows each, which form the running products on the way into LDS: the
+// first DP of 2 DP roles stage q, f and q F, the others k and k B. The products with the state and with v run on the f32
+// matrix cores (16x16x4 tiles); a wave keeps its part of the state in the accumulator layout (tile i, element e: row d =
+// 16 i + 4 gg + e of lane group gg), which is also the B operand of (q F) S. Of the 16 x 16 weights of the second sum the
+// block t >= 8 > j is such a product too, with the decays split at row 8 (both factors are the lanes' own running
+// products); the two 8 x 8 blocks on the diagonal are formed on the vector units while the matrix cores are busy: 32
+// lanes per row t share its channels, and q_t times the decays so far is carried down j. Rows past the sequence have f = 1,
+// k = q = 0. D <= 16 NT, NT even.
 template <typename T, int NT>
-__global__ __launch_bounds__(256) void forget_chunk_kernel(const T* __restrict__ q, long q_ld, const T* __restrict__ z,
+__global__ __launch_bounds__(512, NT <= 8 ? 4 : 2) void forget_chunk_kernel(const T* __restrict__ q, long q_ld, const T* __restrict__ z,
                                                            long z_ld, const T* __restrict__ v, long v_ld,
                                                            const float* __restrict__ f_bias,
                                                            const float* __restrict__ lower, float* __restrict__ state,
@@ -55,80 +64,85 @@ __global__ __launch_bounds__(256) void forget_chunk_kernel(const T* __restrict__
                                                            const int* __restrict__ row_cu,
                                                            const int* __restrict__ positions, int act, int vec,
                                                            float* __restrict__ o, int H, int D, int Dv) {
-  constexpr int C = 16, DP = 16 * NT, NU = (DP + 63) / 64, KP = 64 * NU + 4, VP = 68, PP = C + 4;
-  constexpr int NI = (2 * DP + 255) / 256;
-  constexpr bool FAST = sizeof(T) == 2;
+  constexpr int C = 16, DP = 16 * NT, NH = NT / 2, NU = (DP + 127) / 128, KP = 128 * NU + 4, VP = 68, PP = C + 4;
+  constexpr int NI = (2 * DP + 255) / 256, HC = C / 2, NP = NT < 8 ? NT : 8;
+  constexpr bool FAST = sizeof(T) == 2, WHOLE = NI * 256 == 2 * DP;
   extern __shared__ __attribute__((aligned(16))) float smem[];
   float* sq = smem;                     // [C][KP] q
   float* sk = sq + C * KP;              // [C][KP] k
   float* sf = sk + C * KP;              // [C + 1][KP] f; row C holds ones
   float* sqf = sf + (C + 1) * KP;       // [C][KP] q F
   float* skb = sqf + C * KP;            // [C][KP] k B
-  float* sv = skb + C * KP;             // [C][VP]
-  float* sp = sv + C * VP;              // [C][PP]
-  float* sl = sp + C * PP;              // [DP] F of the last row
+  float* sqh = skb + C * KP;            // [HC][KP] q times the decays from row 8 on, of rows 8 .. 15
+  float* skh = sqh + HC * KP;           // [HC][KP] k times the decays up to row 7, of rows 0 .. 7
+  float* sv = skh + HC * KP;            // [C][VP]
+  float* so = sv + C * VP;              // [C][VP] (q F) S over the second half of the state's rows
+  float* sp = so + C * VP;              // [C][PP] weights; those of rows 8 .. 15 on columns 0 .. 7 come as the sum of
+  float* sph = sp + C * PP;             // [NP][HC][HC] the waves' parts
+  float* sl = sph + NP * HC * HC;       // [DP] F of the last row
   const int s = blockIdx.x, h = blockIdx.y, c0 = blockIdx.z * 64;
   const int r0 = __builtin_amdgcn_readfirstlane(row_cu[s]), r1 = __builtin_amdgcn_readfirstlane(row_cu[s + 1]);
   if (r1 <= r0) return;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, m = lane & 15, gg = lane >> 4;
   const int slot = state_slots[s];
   if (slot < 0) {      // padding sequence of a fixed-shape step: defined output, no state
-    for (int i = tid; i < (r1 - r0) * 64; i += 256)
+    for (int i = tid; i < (r1 - r0) * 64; i += 512)
       if (c0 + (i & 63) < Dv) o[((long)(r0 + (i >> 6)) * H + h) * Dv + c0 + (i & 63)] = 0.f;
     return;
   }
-  const int cl = 16 * wave + m, col = c0 + cl;
+  const int cl = 16 * (wave & 3) + m, col = c0 + cl, d0 = (wave >> 2) * 16 * NH;
   const bool live = col < Dv;
   float* S = state + ((long)slot * H + h) * D * Dv + col;
   const bool fresh = positions[r0] == 0;
-  f32x4 st[NT];
+  f32x4 st[NH];
 #pragma unroll
-  for (int i = 0; i < NT; ++i)
+  for (int i = 0; i < NH; ++i)
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
-      const int d = 16 * i + 4 * gg + e;
+      const int d = d0 + 16 * i + 4 * gg + e;
       st[i][e] = (!fresh && live && d < D) ? S[(long)d * Dv] : 0.f;
     }
-  for (int i = tid; i < KP; i += 256) sf[C * KP + i] = 1.f;
-  if (DP < 64 * NU) {      // columns that no role stages
-    constexpr int R = 64 * NU - DP > 0 ? 64 * NU - DP : 1;
-    for (int i = tid; i < C * R; i += 256) {
+  for (int i = tid; i < KP; i += 512) sf[C * KP + i] = 1.f;
+  if (tid < HC * HC) sp[(tid / HC) * PP + HC + tid % HC] = 0.f;      // (above the diagonal blocks, never written again)
+  if (DP < 128 * NU) {      // columns that no role stages
+    constexpr int R = 128 * NU - DP > 0 ? 128 * NU - DP : 1;
+    for (int i = tid; i < C * R; i += 512) {
       const int at = (i / R) * KP + DP + i % R;
       sq[at] = sk[at] = 0.f;
       sf[at] = 1.f;
     }
   }
-  // this thread's roles: channel, bias and lower bound (channels past D: k = q = 0, f = 1)
+  // this thread's roles: channel, rows ra .. ra + 7, bias and lower bound
+  const int role = 32 * wave + (lane & 31), hf = lane >> 5, ra = HC * hf;
   float rb[NI], rl[NI];
 #pragma unroll
   for (int u = 0; u < NI; ++u) {
-    const int idx = tid + 256 * u, d = min(idx < DP ? idx : idx - DP, D - 1);
+    const int idx = role + 256 * u, d = min(idx < DP ? idx : idx - DP, D - 1);
     rb[u] = f_bias[(long)h * D + d];
     rl[u] = lower[(long)h * D + d];
   }
   // the next chunk's inputs as they are stored (rows past the sequence: its last row again)
   typedef T t4 __attribute__((ext_vector_type(4)));
-  T rq[NI][C], rz[NI][C];
+  T rq[NI][HC], rz[NI][HC];
   t4 rv;
   auto fetch = [&](int t0) {
-    // (one descriptor per chunk; a load takes the channel's vector offset and the row's scalar offset)
     const __amdgpu_buffer_rsrc_t qb = rows_rsrc(q + (long)t0 * q_ld + (long)h * D);
     const __amdgpu_buffer_rsrc_t zb = rows_rsrc(z + (long)t0 * z_ld + (long)h * D);
-    const int qs = (int)q_ld * (int)sizeof(T), zs = (int)z_ld * (int)sizeof(T);
-    const int last = r1 - 1 - t0;
+    const int qs = (int)q_ld * (int)sizeof(T), zs = (int)z_ld * (int)sizeof(T), last = r1 - 1 - t0;
 #pragma unroll
     for (int u = 0; u < NI; ++u) {
-      const int idx = tid + 256 * u;
+      const int idx = role + 256 * u;
       const int d = min(idx < DP ? idx : idx - DP, D - 1) * (int)sizeof(T);
       if (idx < DP) {
 #pragma unroll
-        for (int i = 0; i < C; ++i) rq[u][i] = row_load<T>(qb, d, __builtin_amdgcn_readfirstlane(min(i, last) * qs));
+        for (int i = 0; i < HC; ++i) rq[u][i] = row_load<T>(qb, __umul24(min(ra + i, last), qs) + d);
       }
-      if (NI * 256 == 2 * DP || idx < 2 * DP) {
+      if (WHOLE || idx < 2 * DP) {
 #pragma unroll
-        for (int i = 0; i < C; ++i) rz[u][i] = row_load<T>(zb, d, __builtin_amdgcn_readfirstlane(min(i, last) * zs));
+        for (int i = 0; i < HC; ++i) rz[u][i] = row_load<T>(zb, __umul24(min(ra + i, last), zs) + d);
       }
     }
+    if (tid >= 256) return;
     const T* vr = v + (long)min(t0 + (tid >> 4), r1 - 1) * v_ld + (long)h * Dv;
     const int c = c0 + 4 * (tid & 15);
     if (vec & 2) {
@@ -138,50 +152,70 @@ __global__ __launch_bounds__(256) void forget_chunk_kernel(const T* __restrict__
       for (int e = 0; e < 4; ++e) rv[e] = vr[min(c + e, Dv - 1)];
     }
   };
-  // Gates of this thread's channels into LDS. No branch: a row past the sequence is set to f = 1, k = q = 0 by factors
-  // (`tail`: the last chunk has such rows), a channel past D has q = 0 (its state row is never read or stored).
+  // Gates of this thread's channels into LDS. No branch on rows or channels: a row past the sequence is set to f = 1, k =
+  // q = 0 by factors (`tail`: the last chunk has such rows), a channel past D has q = 0 (its state row is never read or
+  // stored). The running products cross from one half of the rows to the other between lanes l and l + 32.
   auto stage = [&](int n, auto tail) {
 #pragma unroll
     for (int u = 0; u < NI; ++u) {
-      const int idx = tid + 256 * u;
+      const int idx = role + 256 * u;
       const float one = 1.f - rl[u];
       if (idx < DP) {
         const float qm = idx < D ? 1.f : 0.f;
-        float F = 1.f;
+        float F = 1.f, w[HC];
 #pragma unroll
-        for (int i = 0; i < C; ++i) {
-          const float in = decltype(tail)::value ? (i < n ? 1.f : 0.f) : 1.f;
+        for (int i = 0; i < HC; ++i) {
           float sg, cg;
           sigmoid2<FAST>((float)rz[u][i] + rb[u], sg, cg);
           float f = fmaf(one, sg, rl[u]), qv = act_in<FAST>((float)rq[u][i], act) * qm;
           if (decltype(tail)::value) {
+            const float in = ra + i < n ? 1.f : 0.f;
             f = fmaf(in, f, 1.f - in);
             qv *= in;
           }
           F *= f;
-          sq[i * KP + idx] = qv;
-          sf[i * KP + idx] = f;
-          sqf[i * KP + idx] = qv * F;
+          sq[(ra + i) * KP + idx] = qv;
+          sf[(ra + i) * KP + idx] = f;
+          w[i] = qv * F;
         }
-        sl[idx] = F;
-      } else if (NI * 256 == 2 * DP || idx < 2 * DP) {
-        const int d = idx - DP;
-        float B = 1.f;
+        const float Fo = __shfl_xor(F, 32, 64), by = hf ? Fo : 1.f;
 #pragma unroll
-        for (int i = C - 1; i >= 0; --i) {
-          const float in = decltype(tail)::value ? (i < n ? 1.f : 0.f) : 1.f;
+        for (int i = 0; i < HC; ++i) {
+          sqf[(ra + i) * KP + idx] = w[i] * by;
+          if (hf) sqh[i * KP + idx] = w[i];
+        }
+        if (hf == 0) sl[idx] = F * Fo;
+      } else if (WHOLE || idx < 2 * DP) {
+        const int d = idx - DP;
+        float B = 1.f, w[HC];
+#pragma unroll
+        for (int i = HC - 1; i >= 0; --i) {
           float sg, cg;
           sigmoid2<FAST>((float)rz[u][i] + rb[u], sg, cg);
           float f = fmaf(one, sg, rl[u]), k = one * cg;
           if (decltype(tail)::value) {
+            const float in = ra + i < n ? 1.f : 0.f;
             f = fmaf(in, f, 1.f - in);
             k *= in;
           }
-          sk[i * KP + d] = k;
-          skb[i * KP + d] = k * B;
+          sk[(ra + i) * KP + d] = k;
+          w[i] = k * B;
           B *= f;
         }
+        const float Bo = __shfl_xor(B, 32, 64), by = hf ? 1.f : Bo;
+#pragma unroll
+        for (int i = 0; i < HC; ++i) {
+          skb[(ra + i) * KP + d] = w[i] * by;
+          if (!hf) skh[i * KP + d] = w[i];
+        }
       }
+    }
+    if (tid < 256) {
+      const int t = tid >> 4, c = 4 * (tid & 15);
+      f32x4 a;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) a[e] = (t < n && c0 + c + e < Dv) ? (float)rv[e] : 0.f;
+      *reinterpret_cast<f32x4*>(sv + t * VP + c) = a;
     }
   };
   fetch(r0);
@@ -189,84 +223,101 @@ __global__ __launch_bounds__(256) void forget_chunk_kernel(const T* __restrict__
     const int n = min(C, r1 - t0);
     if (n == C) stage(n, std::false_type{});
     else stage(n, std::true_type{});
-    {
-      const int t = tid >> 4, c = 4 * (tid & 15);
-      f32x4 a;
-#pragma unroll
-      for (int e = 0; e < 4; ++e) a[e] = (t < n && c0 + c + e < Dv) ? (float)rv[e] : 0.f;
-      *reinterpret_cast<f32x4*>(sv + t * VP + c) = a;
-    }
     if (t0 + C < r1) fetch(t0 + C);      // in flight during the products below
     __syncthreads();
     // (q F) S, then the new state
-    f32x4 oc = {0.f, 0.f, 0.f, 0.f}, oc1 = {0.f, 0.f, 0.f, 0.f};
+    f32x4 oc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int i = 0; i < NT; ++i) {
-      const f32x4 a = *reinterpret_cast<const f32x4*>(sqf + m * KP + 16 * i + 4 * gg);
+    for (int i = 0; i < NH; ++i) {
+      const f32x4 a = *reinterpret_cast<const f32x4*>(sqf + m * KP + d0 + 16 * i + 4 * gg);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        if (i & 1) oc1 = mfma_f32(a[e], st[i][e], oc1);
-        else oc = mfma_f32(a[e], st[i][e], oc);
-      }
+      for (int e = 0; e < 4; ++e) oc = mfma_f32(a[e], st[i][e], oc);
     }
     float bv[4];
 #pragma unroll
     for (int e = 0; e < 4; ++e) bv[e] = sv[(4 * gg + e) * VP + cl];
 #pragma unroll
-    for (int i = 0; i < NT; ++i) {
-      st[i] *= *reinterpret_cast<const f32x4*>(sl + 16 * i + 4 * gg);
+    for (int i = 0; i < NH; ++i) {
+      st[i] *= *reinterpret_cast<const f32x4*>(sl + d0 + 16 * i + 4 * gg);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) st[i] = mfma_f32(skb[(4 * gg + e) * KP + 16 * i + m], bv[e], st[i]);
+      for (int e = 0; e < 4; ++e) st[i] = mfma_f32(skb[(4 * gg + e) * KP + d0 + 16 * i + m], bv[e], st[i]);
     }
-    // the weights of row t: 16 lanes share its channels, lane j keeps weight (t, j)
+    // weights of rows 8 .. 15 on columns 0 .. 7: this wave's channels
+    if (wave < NP) {
+      f32x4 w = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int i = 0; i < (NT + 7) / 8; ++i) {
+        const int at = (m & 7) * KP + 16 * (wave + 8 * i) + 4 * gg;
+        if (NT % 8 && wave + 8 * i >= NT) break;
+        const f32x4 a = *reinterpret_cast<const f32x4*>(sqh + at), b = *reinterpret_cast<const f32x4*>(skh + at);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) w = mfma_f32(a[e], b[e], w);
+      }
+      if (m < HC && gg < 2) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) sph[(wave * HC + 4 * gg + e) * HC + m] = w[e];
+      }
+    }
+    // the diagonal blocks: rows tb and 8 + tb, 32 lanes each share the row's channels, lane 16 + j keeps column j
     {
-      const int t = wave + 4 * gg;
+      const int tb = wave < 4 ? wave : 11 - wave, l4 = 4 * (lane & 31);      // (SIMDs get rows of equal work)
       f32x4 qd[NU];
 #pragma unroll
-      for (int u = 0; u < NU; ++u) qd[u] = *reinterpret_cast<const f32x4*>(sq + t * KP + 64 * u + 4 * m);
+      for (int u = 0; u < NU; ++u) qd[u] = *reinterpret_cast<const f32x4*>(sq + (ra + tb) * KP + 128 * u + l4);
       float keep = 0.f;
 #pragma unroll
-      for (int j = C - 1; j >= 0; --j) {
-        const float* fr = sf + (j < t ? j + 1 : C) * KP + 4 * m;      // (rows at or above t: not decayed yet)
-        const float* kr = sk + j * KP + 4 * m;
-        f32x4 w = {0.f, 0.f, 0.f, 0.f};
+      for (int j = HC - 1; j >= 0; --j) {
+        if (j > tb) continue;
+        const float* fr = sf + (j < tb ? ra + j + 1 : C) * KP + l4;      // (its own column: not decayed yet)
+        const float* kr = sk + (ra + j) * KP + l4;
+        float w = 0.f;
 #pragma unroll
         for (int u = 0; u < NU; ++u) {
-          qd[u] *= *reinterpret_cast<const f32x4*>(fr + 64 * u);
-          const f32x4 kk = *reinterpret_cast<const f32x4*>(kr + 64 * u);
+          qd[u] *= *reinterpret_cast<const f32x4*>(fr + 128 * u);
+          const f32x4 kk = *reinterpret_cast<const f32x4*>(kr + 128 * u);
 #pragma unroll
-          for (int e = 0; e < 4; ++e) w[e] = fmaf(qd[u][e], kk[e], w[e]);
+          for (int e = 0; e < 4; ++e) w = fmaf(qd[u][e], kk[e], w);
         }
-        const float a = row16_sum((w[0] + w[1]) + (w[2] + w[3]));
-        keep = (m == j && j <= t) ? a : keep;
+        w = half_sum(w);
+        keep = m == j ? w : keep;
       }
-      sp[t * PP + m] = keep;
+      if ((lane & 16) && m < HC) sp[(ra + tb) * PP + ra + m] = keep;
+    }
+    if (wave >= 4) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) so[(4 * gg + e) * VP + cl] = oc[e];
     }
     __syncthreads();
-    {
-      const f32x4 a = *reinterpret_cast<const f32x4*>(sp + m * PP + 4 * gg);
+    if (wave < 4) {
+      f32x4 a = *reinterpret_cast<const f32x4*>(sp + m * PP + 4 * gg);
+      if (m >= HC && gg < 2) {
+        a = *reinterpret_cast<const f32x4*>(sph + (m - HC) * HC + 4 * gg);
+#pragma unroll
+        for (int i = 1; i < NP; ++i) a += *reinterpret_cast<const f32x4*>(sph + (i * HC + m - HC) * HC + 4 * gg);
+      }
+#pragma unroll
+      for (int e = 0; e < 4; ++e) oc[e] += so[(4 * gg + e) * VP + cl];
 #pragma unroll
       for (int e = 0; e < 4; ++e) oc = mfma_f32(a[e], bv[e], oc);
-    }
-    oc += oc1;
-    if (live) {
+      if (live) {
 #pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        const int t = 4 * gg + e;
-        if (t < n) o[((long)(t0 + t) * H + h) * Dv + col] = oc[e];
+        for (int e = 0; e < 4; ++e) {
+          const int t = 4 * gg + e;
+          if (t < n) o[((long)(t0 + t) * H + h) * Dv + col] = oc[e];
+        }
       }
     }
-    // (the next chunk's staging writes nothing that is read after the barrier above but sp, which is rewritten only
+    // (the next chunk's staging writes nothing that is read after the barrier above; sp, sph and so are rewritten only
     // after its own first barrier)
   }
   int De = D;
   asm volatile("" : "+s"(De));      // (the bounds are compared anew: kept masks would fill the scalar registers)
   if (live) {
 #pragma unroll
-    for (int i = 0; i < NT; ++i)
+    for (int i = 0; i < NH; ++i)
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
-        const int d = 16 * i + 4 * gg + e;
+        const int d = d0 + 16 * i + 4 * gg + e;
         if (d < De) S[(long)d * Dv] = st[i][e];
       }
   }
@@ -399,8 +450,8 @@ template <typename T, int NT>
 void forget_chunk_launch(const T* q, long q_ld, const T* z, long z_ld, const T* v, long v_ld, const float* f_bias,
                          const float* lower, float* state, const int* state_slots, const int* row_cu, int nseq,
                          const int* positions, int act, int vec, float* o, int H, int D, int Dv, hipStream_t s) {
-  constexpr int DP = 16 * NT, KP = (DP + 63) / 64 * 64 + 4;
-  constexpr size_t lds = (size_t)(81 * KP + 16 * 68 + 16 * 20 + DP) * sizeof(float);
+  constexpr int DP = 16 * NT, KP = (DP + 127) / 128 * 128 + 4;
+  constexpr size_t lds = (size_t)(97 * KP + 2 * 16 * 68 + 16 * 20 + 64 * (NT < 8 ? NT : 8) + DP) * sizeof(float);
   static bool once = false;
   if (!once) {
     (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&forget_chunk_kernel<T, NT>),
@@ -408,7 +459,7 @@ void forget_chunk_launch(const T* q, long q_ld, const T* z, long z_ld, const T* 
     once = true;
   }
   dim3 grid(nseq, H, (Dv + 63) / 64);
-  forget_chunk_kernel<T, NT><<<grid, 256, lds, s>>>(q, q_ld, z, z_ld, v, v_ld, f_bias, lower, state, state_slots, row_cu,
+  forget_chunk_kernel<T, NT><<<grid, 512, lds, s>>>(q, q_ld, z, z_ld, v, v_ld, f_bias, lower, state, state_slots, row_cu,
                                                     positions, act, vec, o, H, D, Dv);
 }
 
