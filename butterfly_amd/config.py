@@ -276,8 +276,8 @@ class ModelConfig:
     @classmethod
     def from_rumedra(cls, js: dict, name: str = "rumedra") -> "ModelConfig":
         """Map a Rumedra config.json ("architecture": "Rumedra") to ModelConfig: pre-norm layers over two
-        mixers (rotated windowed attention beside retention, "parallel"; linear attention whose forget gate
-        also decides what is written, "hgrn2"), dense ReLU GLUs or routed silu GLUs chosen inside the best
+        mixers (rotated windowed attention beside retention, "parallel"; linear attention with a gate per
+        channel as decay and its complement as key, "hgrn2"), dense ReLU GLUs or routed silu GLUs chosen inside the best
         groups of experts, with identity experts and a shared one, a scaled embedding whose table is also the
         LM head. Every size and per-layer constant is taken from the file."""
         kinds = {"parallel": "attention_retention", "hgrn2": "hgrn"}

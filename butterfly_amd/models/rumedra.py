@@ -7,8 +7,8 @@
                         rescaled by wavelength), a sliding window, an ordinary softmax, an elementwise sigmoid
                         gate. Right: linear attention with one constant decay per head (retention), queries
                         and keys half-rotated, keys times dim^(-1/2), unit RMS per head, a silu gate
-    mixer "hgrn"      : linear attention whose decay per channel f = l + (1 - l) sigmoid(W_f h + b) also decides
-                        what is written, S <- diag(f) S + (1 - f) v^T, o = S^T silu(q), RMS norm per head
+    mixer "hgrn"      : linear attention with a decay per channel f = l + (1 - l) sigmoid(W_f h + b) and the key
+                        1 - f, S <- diag(f) S + (1 - f) v^T, o = S^T silu(q), RMS norm per head
     feed-forward      : dense ReLU GLU, or routed silu GLUs: f32 softmax scores, chosen with a correction among
                         the best groups of experts, identity experts that hand on their input, a shared expert
   output      : RMS norm, logits = table x, f32

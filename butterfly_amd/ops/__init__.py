@@ -1369,7 +1369,7 @@ def decay_scan(q, k, v, dpow, state, state_slots, row_cu, positions, act: str = 
 
 
 def forget_scan(q, z, v, f_bias, lower, state, state_slots, row_cu, positions, act: str = "silu", one_row: bool = False):
-    """Linear attention whose decay per head and channel also decides what is written, over packed rows: f = lower +
+    """Linear attention with a gate per head and channel as decay, its complement as key, over packed rows: f = lower +
     (1 - lower) sigmoid(z + f_bias), S <- diag(f) S + (1 - f) v^T, o = S^T act(q), the state pooled as in decay_scan. q, z
     [T, H, D], v [T, H, Dv] rows (views allowed); f_bias, lower [H * D] f32. Steps of several rows per sequence run
     in chunks of 16 rows on the f32 matrix cores, steps of one row (`one_row`) in place. Returns o [T, H,

@@ -1,4 +1,4 @@
-// Linear attention whose decay per head and channel also decides what is written, and the norm per head that
+// Linear attention with a gate per head and channel as decay and its complement as key, and the norm per head that
 // follows a linear attention; generic in every size and in the activation type (bf16 or f32; gates, decays, states
 // and the recurrence are f32 in both):
 //   forget_chunk_kernel, forget_step_kernel   f = l + (1 - l) sigmoid(z + b), S <- diag(f) S + (1 - f) v^T, o = S^T q,
